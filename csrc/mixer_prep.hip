@@ -6,6 +6,10 @@
 //                    of the queries' rotary parts, paged append of
 //                    [latent | key part], assembly of the latent-space
 //                    queries;
+//   rms_norm_rows    rows over their root mean square, times a weight (the
+//                    latent a query passes);
+//   merge_heads      per-head outputs side by side, each head times the
+//                    sigmoid of its gate;
 //   pool_append      mean key/value of every block of positions a step
 //                    completes, into the pooled caches;
 //   short_conv_silu  causal per-channel convolution over time + silu with
@@ -244,6 +248,50 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
           q[(size_t)t * ldq + h * (D + R) + D + R - 1];
 }
 
+// y[t] = x[t] / sqrt(mean(x[t]^2) + eps) * w. One workgroup per row.
+template <typename T>
+__global__ __launch_bounds__(256) void rms_norm_rows_kernel(
+    T* __restrict__ y, const T* __restrict__ x, int ldx,
+    const float* __restrict__ w, float eps, int C) {
+  __shared__ float red[17];
+  const T* xr = x + (size_t)blockIdx.x * ldx;
+  T* yr = y + (size_t)blockIdx.x * C;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < C; c += blockDim.x) {
+    const float v = MxElem<T>::ld(xr + c);
+    ss += v * v;
+  }
+  const float inv = 1.0f / sqrtf(mx_block_sum(ss, red) / (float)C + eps);
+  for (int c = threadIdx.x; c < C; c += blockDim.x)
+    MxElem<T>::st(yr + c, MxElem<T>::ld(xr + c) * inv * w[c]);
+}
+
+// out[t, h*DV + d] = o[h][t][d] * sigmoid(gate[t, h]) (gate nullptr: the
+// plain copy). Grid (column chunks, tokens); a thread takes V consecutive
+// entries of one head (V divides DV).
+template <typename T, int V>
+__global__ __launch_bounds__(256) void merge_heads_kernel(
+    T* __restrict__ out, int ldo, const T* __restrict__ o,
+    const T* __restrict__ gate, int ldg, int T_, int H, int DV) {
+  const int t = blockIdx.y;
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (c >= H * DV) return;
+  const int h = c / DV, d = c - h * DV;
+  const T* src = o + ((size_t)h * T_ + t) * DV + d;
+  T* dst = out + (size_t)t * ldo + c;
+  const float g = gate != nullptr
+                      ? mx_sigmoid(MxElem<T>::ld(gate + (size_t)t * ldg + h))
+                      : 1.f;
+  struct __align__(sizeof(T) * V) Vec {
+    T e[V];
+  };
+  const Vec v = *(const Vec*)src;
+  Vec r;
+#pragma unroll
+  for (int i = 0; i < V; ++i) MxElem<T>::st(&r.e[i], MxElem<T>::ld(&v.e[i]) * g);
+  *(Vec*)dst = r;
+}
+
 // Thread = channel, workgroup = (channel tile, segment, chunk of CONV_CH
 // tokens). A thread keeps the K-1 inputs before its current token in
 // registers. Only chunk 0 of a segment reads the sequence's state, and it
@@ -365,6 +413,37 @@ void mx_latent_prep(void* qf, const void* qlat, const void* q, int ldq,
                        (const float*)normw, eps, (const float*)cos_sin,
                        table_rows, rot_dims, (const int*)positions,
                        (T*)cache, (const int64_t*)slots, T_, H, D, R, L, BS);
+  })
+}
+
+void mx_rms_norm_rows(void* y, const void* x, int ldx, const void* w,
+                      float eps, int T_, int C, int dtype, void* stream) {
+  if (T_ <= 0 || C <= 0) return;
+  MX_DISPATCH_DTYPE(dtype, {
+    hipLaunchKernelGGL((rms_norm_rows_kernel<T>), dim3(T_), dim3(256), 0,
+                       (hipStream_t)stream, (T*)y, (const T*)x, ldx,
+                       (const float*)w, eps, C);
+  })
+}
+
+void mx_merge_heads(void* out, int ldo, const void* o, const void* gate,
+                    int ldg, int T_, int H, int DV, int dtype,
+                    void* stream) {
+  if (T_ <= 0 || H * DV <= 0) return;
+  const bool aligned = (((size_t)out | (size_t)o) & 15) == 0;
+  MX_DISPATCH_DTYPE(dtype, {
+    constexpr int V = 16 / sizeof(T);
+    if (aligned && DV % V == 0 && ldo % V == 0) {
+      hipLaunchKernelGGL((merge_heads_kernel<T, V>),
+                         dim3((H * DV / V + 255) / 256, T_), dim3(256), 0,
+                         (hipStream_t)stream, (T*)out, ldo, (const T*)o,
+                         (const T*)gate, ldg, T_, H, DV);
+    } else {
+      hipLaunchKernelGGL((merge_heads_kernel<T, 1>),
+                         dim3((H * DV + 255) / 256, T_), dim3(256), 0,
+                         (hipStream_t)stream, (T*)out, ldo, (const T*)o,
+                         (const T*)gate, ldg, T_, H, DV);
+    }
   })
 }
 

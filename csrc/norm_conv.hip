@@ -12,6 +12,11 @@
 //                      the ragged batch, the segment's previous K - 1 normed
 //                      rows coming from (and its last K - 1 going to) fp32
 //                      per-sequence state.
+// EXT instantiations of the first kernel: the one delta is also multiplied,
+// element by element, by sigmoid(z + zb) (a gated residual branch); and for
+// steps whose segments are all single rows the convolution runs in the same
+// launch, since it then needs nothing but the row itself and the sequence's
+// state.
 // Splitting at the row statistics keeps the stream's extra traffic to one
 // re-read: neighbouring rows' normed values are recomputed from registers,
 // never stored.
@@ -43,13 +48,52 @@ PS_DEV void nc_st4(mx_bf16* p, const float4& v) {
 // NC_Q entries, and all rows start 16-byte aligned: a thread then keeps its
 // entries (four at a time) in registers between the passes.
 #define NC_Q 8
+#define NC_MAX_TAPS 32
 
-template <typename TD, typename TO, bool VEC>
+// Options of the EXT form; pointers are nullptr where an option is off.
+template <typename TO>
+struct NcExt {
+  const TO* z;          // [T, W] residual gate before bias and sigmoid
+  int ldz;
+  const float* zb;      // [W]
+  TO* yp;               // [T, W] normed rows before the convolution
+  const float* cw;      // [W, K] convolution of single-row segments
+  float* state;         // [slots, K - 1, W]
+  const int* seq_rows;  // segment t is row t
+  int K;
+};
+
+// Convolution of a single-row segment, N consecutive channels from c on:
+// acc[i] += conv(y)[c + i]; the state moves on by one row.
+template <int N>
+PS_DEV void nc_single(const float* __restrict__ cw, float* __restrict__ state,
+                      const int* __restrict__ sr, int K, int W, int c,
+                      const float* y, float* acc) {
+  const bool past = sr[2] > 0;
+  float* st = state + (size_t)sr[3] * (K - 1) * W + c;
+  float old[N];
+#pragma unroll
+  for (int i = 0; i < N; ++i) acc[i] += cw[(size_t)(c + i) * K + K - 1] * y[i];
+  for (int j = 0; j < K - 1; ++j) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) old[i] = past ? st[(size_t)j * W + i] : 0.f;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      acc[i] += cw[(size_t)(c + i) * K + j] * old[i];
+      if (j > 0) st[(size_t)(j - 1) * W + i] = old[i];
+    }
+  }
+  if (K > 1)
+#pragma unroll
+    for (int i = 0; i < N; ++i) st[(size_t)(K - 2) * W + i] = y[i];
+}
+
+template <typename TD, typename TO, bool VEC, bool EXT>
 __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
     TO* __restrict__ h, float* __restrict__ x, const TD* __restrict__ d0,
     int ld0, float s0, const TD* __restrict__ d1, int ld1, float s1,
     const float* __restrict__ w, const float* __restrict__ b, float eps,
-    float* __restrict__ stats, int W) {
+    float* __restrict__ stats, int W, NcExt<TO> ext) {
   __shared__ float red[17];
   const int t = blockIdx.x;
   float* xr = x + (size_t)t * W;
@@ -62,7 +106,15 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
       if (c < W) {
         v[i] = nc_ld4(xr + c);
         if (d0 != nullptr) {
-          const float4 a = nc_ld4(d0 + (size_t)t * ld0 + c);
+          float4 a = nc_ld4(d0 + (size_t)t * ld0 + c);
+          if (EXT && ext.z != nullptr) {
+            const float4 z = nc_ld4(ext.z + (size_t)t * ext.ldz + c);
+            const float4 zb = nc_ld4(ext.zb + c);
+            a.x *= mx_sigmoid(z.x + zb.x);
+            a.y *= mx_sigmoid(z.y + zb.y);
+            a.z *= mx_sigmoid(z.z + zb.z);
+            a.w *= mx_sigmoid(z.w + zb.w);
+          }
           v[i].x += s0 * a.x;
           v[i].y += s0 * a.y;
           v[i].z += s0 * a.z;
@@ -106,6 +158,14 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
           o.y = (v[i].y - mean) * rstd * ww.y + bb.y;
           o.z = (v[i].z - mean) * rstd * ww.z + bb.z;
           o.w = (v[i].w - mean) * rstd * ww.w + bb.w;
+          if (EXT && ext.cw != nullptr) {
+            if (ext.yp != nullptr) nc_st4(ext.yp + (size_t)t * W + c, o);
+            const float y[4] = {o.x, o.y, o.z, o.w};
+            float acc[4] = {o.x, o.y, o.z, o.w};
+            nc_single<4>(ext.cw, ext.state, ext.seq_rows + 4 * t, ext.K, W, c,
+                         y, acc);
+            o = make_float4(acc[0], acc[1], acc[2], acc[3]);
+          }
           nc_st4(h + (size_t)t * W + c, o);
         }
       }
@@ -117,6 +177,9 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
     float v = xr[c];
     if (d0 != nullptr) {
       float d = s0 * MxElem<TD>::ld(d0 + (size_t)t * ld0 + c);
+      if (EXT && ext.z != nullptr)
+        d *= mx_sigmoid(MxElem<TO>::ld(ext.z + (size_t)t * ext.ldz + c) +
+                        ext.zb[c]);
       if (d1 != nullptr) d += s1 * MxElem<TD>::ld(d1 + (size_t)t * ld1 + c);
       v += d;
       xr[c] = v;
@@ -136,9 +199,16 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
     stats[2 * t + 1] = rstd;
   }
   if (h != nullptr)
-    for (int c = threadIdx.x; c < W; c += blockDim.x)
-      MxElem<TO>::st(h + (size_t)t * W + c,
-                     (xr[c] - mean) * rstd * w[c] + b[c]);
+    for (int c = threadIdx.x; c < W; c += blockDim.x) {
+      const float y = (xr[c] - mean) * rstd * w[c] + b[c];
+      float acc = y;
+      if (EXT && ext.cw != nullptr) {
+        if (ext.yp != nullptr) MxElem<TO>::st(ext.yp + (size_t)t * W + c, y);
+        nc_single<1>(ext.cw, ext.state, ext.seq_rows + 4 * t, ext.K, W, c, &y,
+                     &acc);
+      }
+      MxElem<TO>::st(h + (size_t)t * W + c, acc);
+    }
 }
 
 // A workgroup takes 256 channels of up to NC_ROWS consecutive rows of one
@@ -149,12 +219,12 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
 #define NC_ROWS 64
 
 // KT: taps at compile time; 0: `taps` of them (up to NC_MAX_TAPS), with the
-// window in arrays of that size.
-#define NC_MAX_TAPS 32
+// window in arrays of that size. yp: the normed rows before the convolution
+// are stored there too (nullptr: not).
 
 template <typename TO, int KT>
 __global__ __launch_bounds__(256) void norm_conv32_kernel(
-    TO* __restrict__ h, const float* __restrict__ x,
+    TO* __restrict__ h, TO* __restrict__ yp, const float* __restrict__ x,
     const float* __restrict__ stats, const float* __restrict__ w,
     const float* __restrict__ b, const float* __restrict__ cw,
     float* __restrict__ state, const int* __restrict__ seq_rows, int W,
@@ -197,6 +267,7 @@ __global__ __launch_bounds__(256) void norm_conv32_kernel(
     for (int j = 0; j + 1 < K - 1; ++j) win[j] = win[j + 1];
     if (K > 1) win[K - 2] = cur;
     MxElem<TO>::st(h + (size_t)t * W + c, acc);
+    if (yp != nullptr) MxElem<TO>::st(yp + (size_t)t * W + c, cur);
   }
   if (a == 0) {
     // old[] holds the previous state (rows -(K-1) .. -1 of the segment)
@@ -221,29 +292,41 @@ __global__ __launch_bounds__(256) void norm_conv32_kernel(
 
 extern "C" {
 
-void mx_add_layer_norm32(void* h, void* x, const void* d0, int ld0, float s0,
-                         const void* d1, int ld1, float s1, const void* w,
-                         const void* b, float eps, void* stats, int T_, int W,
-                         int delta_dtype, int out_dtype, void* stream) {
-  if (T_ <= 0) return;
+// Returns 1 when the taps are not built.
+int mx_add_layer_norm32(void* h, void* x, const void* d0, int ld0, float s0,
+                        const void* d1, int ld1, float s1, const void* w,
+                        const void* b, float eps, void* stats, int T_, int W,
+                        int delta_dtype, int out_dtype, const void* z,
+                        int ldz, const void* zb, void* yp, const void* cw,
+                        void* state, const void* seq_rows, int K,
+                        void* stream) {
+  if (T_ <= 0) return 0;
+  if (cw != nullptr && (K < 1 || K > NC_MAX_TAPS)) return 1;
   // four entries per load: whole vectors per row, aligned row starts
   const bool vec =
       W % 4 == 0 && W <= 1024 * NC_Q && ld0 % 4 == 0 && ld1 % 4 == 0 &&
+      ldz % 4 == 0 &&
       (((size_t)h | (size_t)x | (size_t)d0 | (size_t)d1 | (size_t)w |
-        (size_t)b) & 15) == 0;
+        (size_t)b | (size_t)z | (size_t)zb | (size_t)yp) & 15) == 0;
+  const bool e = z != nullptr || cw != nullptr;
+#define ALN_K(TD, TO, VEC, EXT)                                              \
+  hipLaunchKernelGGL((add_layer_norm32_kernel<TD, TO, VEC, EXT>), dim3(T_),  \
+                     dim3(256), 0, (hipStream_t)stream, (TO*)h, (float*)x,   \
+                     (const TD*)d0, ld0, s0, (const TD*)d1, ld1, s1,         \
+                     (const float*)w, (const float*)b, eps, (float*)stats,   \
+                     W,                                                      \
+                     (NcExt<TO>{(const TO*)z, ldz, (const float*)zb,         \
+                                (TO*)yp, (const float*)cw, (float*)state,    \
+                                (const int*)seq_rows, K}))
 #define ALN_GO(TD, TO)                                                       \
-  if (vec)                                                                   \
-    hipLaunchKernelGGL((add_layer_norm32_kernel<TD, TO, true>), dim3(T_),    \
-                       dim3(256), 0, (hipStream_t)stream, (TO*)h, (float*)x, \
-                       (const TD*)d0, ld0, s0, (const TD*)d1, ld1, s1,       \
-                       (const float*)w, (const float*)b, eps, (float*)stats, \
-                       W);                                                   \
+  if (vec && e)                                                              \
+    ALN_K(TD, TO, true, true);                                               \
+  else if (vec)                                                              \
+    ALN_K(TD, TO, true, false);                                              \
+  else if (e)                                                                \
+    ALN_K(TD, TO, false, true);                                              \
   else                                                                       \
-    hipLaunchKernelGGL((add_layer_norm32_kernel<TD, TO, false>), dim3(T_),   \
-                       dim3(256), 0, (hipStream_t)stream, (TO*)h, (float*)x, \
-                       (const TD*)d0, ld0, s0, (const TD*)d1, ld1, s1,       \
-                       (const float*)w, (const float*)b, eps, (float*)stats, \
-                       W)
+    ALN_K(TD, TO, false, false)
   if (delta_dtype == MX_BF16) {
     if (out_dtype == MX_BF16) {
       ALN_GO(mx_bf16, mx_bf16);
@@ -258,19 +341,21 @@ void mx_add_layer_norm32(void* h, void* x, const void* d0, int ld0, float s0,
     }
   }
 #undef ALN_GO
+#undef ALN_K
+  return 0;
 }
 
 #define NC_CASE(KK)                                                          \
   case KK:                                                                   \
     hipLaunchKernelGGL((norm_conv32_kernel<T, KK>), grid, dim3(256), 0,      \
-                       (hipStream_t)stream, (T*)h, (const float*)x,          \
+                       (hipStream_t)stream, (T*)h, (T*)yp, (const float*)x,  \
                        (const float*)stats, (const float*)w,                 \
                        (const float*)b, (const float*)cw, (float*)state,     \
                        (const int*)seq_rows, W, K);                          \
     break;
 
-int mx_norm_conv32(void* h, const void* x, const void* stats, const void* w,
-                   const void* b, const void* cw, void* state,
+int mx_norm_conv32(void* h, void* yp, const void* x, const void* stats,
+                   const void* w, const void* b, const void* cw, void* state,
                    const void* seq_rows, int S_, int W, int K, int T_,
                    int dtype, void* stream) {
   if (S_ <= 0 || T_ <= 0) return 0;
@@ -290,8 +375,9 @@ int mx_norm_conv32(void* h, const void* x, const void* stats, const void* w,
       NC_CASE(8)
       default:
         hipLaunchKernelGGL((norm_conv32_kernel<T, 0>), grid, dim3(256), 0,
-                           (hipStream_t)stream, (T*)h, (const float*)x,
-                           (const float*)stats, (const float*)w,
+                           (hipStream_t)stream, (T*)h, (T*)yp,
+                           (const float*)x, (const float*)stats,
+                           (const float*)w,
                            (const float*)b, (const float*)cw, (float*)state,
                            (const int*)seq_rows, W, K);
     }

@@ -1,15 +1,27 @@
-// fp32 residual-stream kernels: scaled embedding gather, fused
+// fp32 residual-stream kernels: scaled embedding gather (+ learned position
+// rows), fused
 // (residual += deltas) + (grouped) RMSNorm, grouped RMSNorm + token shift,
-// depth-weighted sum of residual streams, gated-MLP inner activations, paged
+// depth-weighted sum of residual streams, gated-MLP inner activations,
+// polynomial norm activation, paged
 // KV append with independent key/value widths.
 #include "mix_common.h"
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_scale_kernel(
     float* __restrict__ x, const int64_t* __restrict__ tokens,
-    const T* __restrict__ embed, float scale, int W) {
+    const T* __restrict__ embed, float scale, int W,
+    const T* __restrict__ pos, int pos_rows,
+    const int* __restrict__ positions) {
   const int t = blockIdx.x;
   const T* row = embed + (size_t)tokens[t] * W;
+  if (pos != nullptr) {
+    const T* pr =
+        pos + (size_t)min(max(positions[t], 0), pos_rows - 1) * W;
+    for (int c = threadIdx.x; c < W; c += blockDim.x)
+      x[(size_t)t * W + c] =
+          MxElem<T>::ld(row + c) * scale + MxElem<T>::ld(pr + c);
+    return;
+  }
   for (int c = threadIdx.x; c < W; c += blockDim.x)
     x[(size_t)t * W + c] = MxElem<T>::ld(row + c) * scale;
 }
@@ -207,6 +219,94 @@ __global__ __launch_bounds__(256) void gated_act_bf16x8_kernel(
   *(uint4*)(out + (size_t)t * ldo + c) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
 }
 
+// Polynomial norm activation of a row z: with N(v) = v / sqrt(mean(v^2) +
+// eps) over the row, y = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3. One workgroup
+// per row; the three sums of squares (z^2, z^4, z^6) come from one pass.
+// VEC (bf16 rows of whole 16-byte vectors, at most 2048 * PN_Q entries):
+// the row stays in registers between the passes.
+#define PN_Q 8
+
+PS_DEV void pn_block_sum3(float* s, float* red) {
+#pragma unroll
+  for (int i = 0; i < 3; ++i) s[i] = mx_wave_sum(s[i]);
+  const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  if ((threadIdx.x & 63) == 0)
+    for (int i = 0; i < 3; ++i) red[wave * 3 + i] = s[i];
+  __syncthreads();
+  for (int i = 0; i < 3; ++i) {
+    s[i] = 0.f;
+    for (int w = 0; w < nw; ++w) s[i] += red[w * 3 + i];
+  }
+}
+
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void poly_norm_kernel(
+    T* __restrict__ out, int ldo, const T* __restrict__ z, int ldz,
+    const float* __restrict__ coef, float eps, int F) {
+  __shared__ float red[12];
+  const T* zr = z + (size_t)blockIdx.x * ldz;
+  T* yr = out + (size_t)blockIdx.x * ldo;
+  const float c0 = coef[0], c1 = coef[1], c2 = coef[2], c3 = coef[3];
+  float s[3] = {0.f, 0.f, 0.f};
+  if (VEC) {
+    uint4 v[PN_Q];
+#pragma unroll
+    for (int i = 0; i < PN_Q; ++i) {
+      const int c = (threadIdx.x + 256 * i) * 8;
+      if (c < F) {
+        v[i] = *(const uint4*)((const unsigned short*)zr + c);
+        const unsigned int w[4] = {v[i].x, v[i].y, v[i].z, v[i].w};
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+          const float x = __uint_as_float((k & 1) ? (w[k >> 1] & 0xffff0000u)
+                                                  : (w[k >> 1] << 16));
+          const float q = x * x;
+          s[0] += q;
+          s[1] += q * q;
+          s[2] += q * q * q;
+        }
+      }
+    }
+    pn_block_sum3(s, red);
+    const float a = c0 / sqrtf(s[0] / (float)F + eps);
+    const float b = c1 / sqrtf(s[1] / (float)F + eps);
+    const float d = c2 / sqrtf(s[2] / (float)F + eps);
+#pragma unroll
+    for (int i = 0; i < PN_Q; ++i) {
+      const int c = (threadIdx.x + 256 * i) * 8;
+      if (c < F) {
+        const unsigned int w[4] = {v[i].x, v[i].y, v[i].z, v[i].w};
+        unsigned int o[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+          const float x0 = __uint_as_float(w[k] << 16);
+          const float x1 = __uint_as_float(w[k] & 0xffff0000u);
+          const float y0 = x0 * (a + x0 * (b + x0 * d)) + c3;
+          const float y1 = x1 * (a + x1 * (b + x1 * d)) + c3;
+          o[k] = (unsigned int)ps_f32_to_bf16(y0) |
+                 ((unsigned int)ps_f32_to_bf16(y1) << 16);
+        }
+        *(uint4*)((unsigned short*)yr + c) = make_uint4(o[0], o[1], o[2], o[3]);
+      }
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < F; c += blockDim.x) {
+    const float x = MxElem<T>::ld(zr + c), q = x * x;
+    s[0] += q;
+    s[1] += q * q;
+    s[2] += q * q * q;
+  }
+  pn_block_sum3(s, red);
+  const float a = c0 / sqrtf(s[0] / (float)F + eps);
+  const float b = c1 / sqrtf(s[1] / (float)F + eps);
+  const float d = c2 / sqrtf(s[2] / (float)F + eps);
+  for (int c = threadIdx.x; c < F; c += blockDim.x) {
+    const float x = MxElem<T>::ld(zr + c);
+    MxElem<T>::st(yr + c, x * (a + x * (b + x * d)) + c3);
+  }
+}
+
 // k [T, G*D] (row stride ldk), v [T, G*DV] -> caches [NB, G, BS, D|DV]
 template <typename T>
 __global__ __launch_bounds__(256) void kv_append_kernel(
@@ -299,12 +399,15 @@ __global__ __launch_bounds__(256) void post_norm_add_norm32_kernel(
 extern "C" {
 
 void mx_embed_scale(void* x, const void* tokens, const void* embed,
-                    float scale, int T_, int W, int dtype, void* stream) {
+                    float scale, int T_, int W, const void* pos,
+                    int pos_rows, const void* positions, int dtype,
+                    void* stream) {
   if (T_ <= 0) return;
   MX_DISPATCH_DTYPE(dtype, {
     hipLaunchKernelGGL((embed_scale_kernel<T>), dim3(T_), dim3(256), 0,
                        (hipStream_t)stream, (float*)x,
-                       (const int64_t*)tokens, (const T*)embed, scale, W);
+                       (const int64_t*)tokens, (const T*)embed, scale, W,
+                       (const T*)pos, pos_rows, (const int*)positions);
   })
 }
 
@@ -415,6 +518,24 @@ void mx_gated_act(void* out, int ldo, const void* gate, int ldg,
                          dim3(256), 0, (hipStream_t)stream, (T*)out, ldo,
                          (const T*)gate, ldg, (const T*)up, ldu, F, limit);
     }
+  })
+}
+
+void mx_poly_norm(void* out, int ldo, const void* z, int ldz,
+                  const void* coef, float eps, int T_, int F, int dtype,
+                  void* stream) {
+  if (T_ <= 0 || F <= 0) return;
+  if (dtype == MX_BF16 && F % 8 == 0 && F <= 2048 * PN_Q && ldo % 8 == 0 &&
+      ldz % 8 == 0 && (((size_t)out | (size_t)z) & 15) == 0) {
+    hipLaunchKernelGGL((poly_norm_kernel<mx_bf16, true>), dim3(T_), dim3(256),
+                       0, (hipStream_t)stream, (mx_bf16*)out, ldo,
+                       (const mx_bf16*)z, ldz, (const float*)coef, eps, F);
+    return;
+  }
+  MX_DISPATCH_DTYPE(dtype, {
+    hipLaunchKernelGGL((poly_norm_kernel<T, false>), dim3(T_), dim3(256), 0,
+                       (hipStream_t)stream, (T*)out, ldo, (const T*)z, ldz,
+                       (const float*)coef, eps, F);
   })
 }
 

@@ -35,7 +35,11 @@ class MixerSpec:
     one cached latent of `kv_rank` entries per token; every head has `dim`
     position-free query/key entries and `rot_dim` rotated ones (the rotated
     key part is shared by the heads); `rot_dims` leading entries of the
-    rotated part turn with base `rot_base`, interleaved pairs.
+    rotated part turn with base `rot_base`, interleaved pairs. `window`
+    limits the visible keys as for "attention"; `q_rank` > 0 sends the
+    queries through a latent of that width of their own (RMS-normalised,
+    learned weight); `head_gate` multiplies every head's output by
+    sigmoid(W_g h)_head.
     kind "general_delta" / "channel_delta": gated delta-rule linear
     recurrences with a per-sequence fp32 state of heads x dim x vdim;
     `decay_rank` is the width of the low-rank decay projection
@@ -115,6 +119,8 @@ class MixerSpec:
     combine: str = "norm_mean"        # norm_mean | weighted (pair)
     left_scale: float = 1.0
     right_scale: float = 1.0
+    q_rank: int = 0
+    head_gate: bool = False
 
 
 @dataclass
@@ -131,15 +137,20 @@ class MlpSpec:
     added to the sum the chosen weights are divided by. `gated` False:
     experts (and the shared expert) are down(act(up x)) without a gate
     branch; `shared_gate` False: the shared expert joins unscaled. act
-    "relu2" is relu(z)^2."""
+    "relu2" is relu(z)^2. score "table": no router, a table of
+    `table_rows` rows gives every token id its `top` experts, each with
+    weight 1 / top. act "poly_norm" (dense, not gated): with N(v) = v over
+    its root mean square, c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, four learned
+    numbers."""
 
     kind: str
     ff: int
-    act: str = "silu"          # silu | gelu_tanh | clamped_swish | relu2
+    # silu | gelu_tanh | clamped_swish | relu2 | poly_norm
+    act: str = "silu"
     limit: float = 0.0
     experts: int = 0
     top: int = 0
-    score: str = "softmax"
+    score: str = "softmax"     # softmax | sigmoid | table
     renormalize: bool = True
     weight_on_input: bool = False
     shared_ff: int = 0
@@ -150,6 +161,7 @@ class MlpSpec:
     renorm_eps: float = 0.0
     gated: bool = True
     shared_gate: bool = True
+    table_rows: int = 0
 
 
 @dataclass
@@ -175,6 +187,12 @@ class LayerSpec:
     # sublayer's normed input h passes as h + conv(h) (0 = none); the last
     # taps - 1 normed inputs of both sublayers are per-sequence state
     input_conv: int = 0
+    # False: only the mixer's input passes the convolution
+    mlp_conv: bool = True
+    # every sublayer's output is multiplied element by element by
+    # sigmoid(W_r h + b_r), h being the sublayer's normed input (before the
+    # input convolution), ahead of joining the residual stream
+    residual_gate: bool = False
 
 
 @dataclass
@@ -219,6 +237,11 @@ class ModelConfig:
     # row with the same weights, every pass with a cache and state of its
     # own; each pass begins with x <- W_in [x; embedding output]
     loop: Optional[tuple] = None
+    # sublayer outputs join the residual stream times this
+    residual_mult: float = 1.0
+    # rows of a learned position table added to the token embeddings
+    # (0 = none): no sequence may be longer
+    learned_positions: int = 0
 
     @property
     def has_recurrent_state(self) -> bool:
@@ -774,6 +797,61 @@ ARCHITECTURES.update({
 })
 
 
+def _lusolix_stack(
+    name: str, width: int, vocab: int, n_layers: int, *, heads: int,
+    dim: int, rot_dim: int, vdim: int, kv_rank: int, q_rank: int,
+    window: int, ff: int, experts: int, top: int, expert_ff: int, taps: int,
+    positions: int, residual_mult: float = 1.0,
+) -> ModelConfig:
+    """A Lusolix stack: windowed latent attention in every layer, a dense
+    feed-forward in the first and table-routed experts in the others; layer
+    norms, an input convolution of `taps` taps ahead of the mixer, gated
+    residual branches, learned positions."""
+    specs = []
+    for i in range(n_layers):
+        mixer = MixerSpec(
+            kind="latent_attention", heads=heads, kv_heads=1, dim=dim,
+            vdim=vdim, kv_rank=kv_rank, q_rank=q_rank, rot_dim=rot_dim,
+            rot_dims=rot_dim, rot_base=500000.0,
+            scale=(dim + rot_dim) ** -0.5, window=window, head_gate=True,
+            rope=True)
+        if i == 0:
+            mlp = MlpSpec(kind="dense", ff=ff, act="poly_norm", gated=False)
+        else:
+            mlp = MlpSpec(kind="moe", ff=expert_ff, act="silu",
+                          experts=experts, top=top, score="table",
+                          renormalize=False, table_rows=vocab)
+        specs.append(LayerSpec(mixer=mixer, mlp=mlp, parallel=False,
+                               norm="layer", input_conv=taps,
+                               mlp_conv=False, residual_gate=True))
+    return ModelConfig(
+        name=name, family="lusolix", hidden_size=width,
+        num_layers=n_layers, num_q_heads=heads, num_kv_heads=1,
+        head_dim=dim + rot_dim, intermediate_size=max(ff, expert_ff),
+        vocab_size=vocab, max_position=positions, layer_specs=specs,
+        residual_mult=residual_mult, learned_positions=positions,
+        tie_word_embeddings=True, bos_token_id=0, eos_token_id=-1)
+
+
+ARCHITECTURES.update({
+    # CPU-runnable test config
+    "tiny-lusolix": _lusolix_stack(
+        "tiny-lusolix", 96, 384, 3, heads=6, dim=16, rot_dim=8, vdim=12,
+        kv_rank=24, q_rank=40, window=24, ff=160, experts=5, top=2,
+        expert_ff=32, taps=3, positions=1024, residual_mult=0.8),
+    # llama-3.2-1b-sized stack (same width, depth, ff and vocab)
+    "lusolix-1b": _lusolix_stack(
+        "lusolix-1b", 2048, 128256, 16, heads=32, dim=64, rot_dim=32,
+        vdim=64, kv_rank=256, q_rank=768, window=1024, ff=8192, experts=8,
+        top=2, expert_ff=2048, taps=4, positions=8192),
+    # llama-3-8b-sized layers (width 4096, head dim 128, ff 14336)
+    "lusolix-8b": _lusolix_stack(
+        "lusolix-8b", 4096, 128256, 32, heads=32, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, q_rank=1536, window=2048, ff=14336,
+        experts=8, top=2, expert_ff=3584, taps=4, positions=8192),
+})
+
+
 @dataclass
 class CacheConfig:
     block_size: int = 16
@@ -876,16 +954,21 @@ class EngineConfig:
             cfg = config_from_dir(self.model)
             if self.weights_path is None:
                 self.weights_path = self.model
-            if self.max_model_len > cfg.max_position:
-                cfg = dataclasses.replace(
-                    cfg, max_position=self.max_model_len)
-            return cfg
+            return self._fit_length(cfg)
         if self.model not in ARCHITECTURES:
             raise ValueError(
                 f"unknown model architecture {self.model!r}; "
                 f"known: {sorted(ARCHITECTURES)}"
             )
-        cfg = ARCHITECTURES[self.model]
+        return self._fit_length(ARCHITECTURES[self.model])
+
+    def _fit_length(self, cfg: ModelConfig) -> ModelConfig:
+        """Computed position codes reach as far as max_model_len asks; a
+        learned position table bounds max_model_len instead (a sequence's
+        last token is never fed, so it may be one longer)."""
+        if cfg.learned_positions:
+            self.max_model_len = min(self.max_model_len,
+                                     cfg.learned_positions + 1)
         if self.max_model_len > cfg.max_position:
             cfg = dataclasses.replace(cfg, max_position=self.max_model_len)
         return cfg

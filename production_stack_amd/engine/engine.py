@@ -168,6 +168,11 @@ class LLMEngine:
                     self.scheduler.add(seq)
                     self.stats.num_requests += 1
                 else:
+                    limit = self.model_cfg.learned_positions
+                    if limit and seq.num_prompt + len(tokens) > limit:
+                        raise ValueError(
+                            f"{rid} grows past the {limit} learned "
+                            "positions")
                     seq.prompt_token_ids.extend(tokens)
                 self.stats.prompt_tokens += len(tokens)
                 plan.append((seq, len(tokens)))

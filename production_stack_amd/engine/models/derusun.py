@@ -348,7 +348,7 @@ class DerusunForCausalLM(nn.Module):
                 cat(mx.in_proj, [mp + "q", mp + "dkv"])
                 put(mx.latent_norm, mp + "dkv.norm")
                 put(mx.uk, mp + "uk")       # [H*dim, L] -> [H, dim, L]
-                put(mx.uv, mp + "uv")       # [H*vdim, L] -> [H, vdim, L]
+                mx.load_uv(f.get_tensor(mp + "uv"))
                 if mx.sink_vals is not None:
                     put(mx.sink_vals, mp + "sink")
             else:

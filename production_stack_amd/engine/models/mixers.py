@@ -211,7 +211,10 @@ class LatentAttention(nn.Module):
     into the latent space (q W_uk), attention runs as single-KV-head
     attention over cached rows [latent | rotary key part] whose values are
     the latent itself, and the result is expanded by W_uv. Only
-    kv_rank + rot_dim numbers per token are cached."""
+    kv_rank + rot_dim numbers per token are cached. `window` limits the
+    visible keys to the trailing ones; with `q_rank` the queries pass a
+    normalised latent of their own; with `head_gate` every head's output is
+    multiplied by the sigmoid of one projected number."""
 
     kind = "latent_attention"
 
@@ -224,12 +227,24 @@ class LatentAttention(nn.Module):
         H, D, R, L = spec.heads, spec.dim, spec.rot_dim, spec.kv_rank
         DV = spec.vdim or D
         self.H, self.D, self.R, self.L, self.DV = H, D, R, L, DV
-        # fused rows: q (per head [dim | rot_dim]) | latent | rotary key
-        self.in_proj = nn.Parameter(
-            torch.empty(H * (D + R) + L + R, width, dtype=dtype))
+        self.q_rank = spec.q_rank
+        # fused rows: q (per head [dim | rot_dim]) or its latent | latent |
+        # rotary key (| head gates)
+        self.q_rows = spec.q_rank or H * (D + R)
+        self.in_proj = nn.Parameter(torch.empty(
+            self.q_rows + L + R + (H if spec.head_gate else 0), width,
+            dtype=dtype))
+        self.q_norm = self.uq = None
+        if spec.q_rank:
+            self.q_norm = nn.Parameter(
+                torch.empty(spec.q_rank, dtype=torch.float32))
+            self.uq = nn.Parameter(
+                torch.empty(H * (D + R), spec.q_rank, dtype=dtype))
         self.latent_norm = nn.Parameter(torch.empty(L, dtype=torch.float32))
         self.uk = nn.Parameter(torch.empty(H, D, L, dtype=dtype))
-        self.uv = nn.Parameter(torch.empty(H, DV, L, dtype=dtype))
+        # transposed against the checkpoint's rows: both folded products
+        # then read a contiguous right operand
+        self.uv = nn.Parameter(torch.empty(H, L, DV, dtype=dtype))
         self.sink_vals = (
             nn.Parameter(torch.empty(H, dtype=torch.float32))
             if spec.learned_sink else None)
@@ -240,6 +255,15 @@ class LatentAttention(nn.Module):
 
     def in_params(self):
         return [self.in_proj]
+
+    def load_uv(self, t: torch.Tensor) -> None:
+        """t: the checkpoint's value up-projection [H * vdim, L]."""
+        H, L, DV = self.H, self.L, self.DV
+        if tuple(t.shape) != (H * DV, L):
+            raise ValueError(
+                f"value up-projection: checkpoint shape {tuple(t.shape)} != "
+                f"{(H * DV, L)}")
+        self.uv.data.copy_(t.to(self.uv.dtype).view(H, DV, L).transpose(1, 2))
 
     @property
     def out_in(self) -> int:
@@ -263,8 +287,11 @@ class LatentAttention(nn.Module):
         sp = self.spec
         T = h.shape[0]
         proj = gemm_policy.linear(h, self.in_proj)
-        q = proj[:, :H * (D + R)]
-        dkv = proj[:, H * (D + R):]
+        q = proj[:, :self.q_rows]
+        dkv = proj[:, self.q_rows:self.q_rows + L + R]
+        if self.q_rank:
+            q = gemm_policy.linear(
+                ops.rms_norm_rows(q, self.q_norm, self.eps), self.uq)
         # position-free query part into the latent space: [H, T, L]
         q_lat = torch.bmm(q.view(T, H, D + R)[:, :, :D].transpose(0, 1),
                           self.uk)
@@ -279,16 +306,13 @@ class LatentAttention(nn.Module):
                 ops.talk_attention(
                     qf[a:b], cache, cache, meta.block_tables,
                     meta.token_seq[a:b], meta.positions[a:b], self.scale, H,
-                    sink=sp.sink, out=o_lat[a:b], variant=variant,
-                    softcap=sp.softcap, sink_vals=self.sink_vals, vdim=L)
+                    window=sp.window, sink=sp.sink, out=o_lat[a:b],
+                    variant=variant, softcap=sp.softcap,
+                    sink_vals=self.sink_vals, vdim=L)
         # expand the attended latents per head: [H, T, L] x [H, L, DV]
-        o = torch.bmm(o_lat.view(T, H, L).transpose(0, 1),
-                      self.uv.transpose(1, 2))
-        o = o.transpose(0, 1).reshape(T, H * DV)
-        if out is not None:
-            out.copy_(o)
-            return out
-        return o
+        o = torch.bmm(o_lat.view(T, H, L).transpose(0, 1), self.uv)
+        gate = proj[:, self.q_rows + L + R:] if sp.head_gate else None
+        return ops.merge_heads(o, gate, out=out)
 
 
 class GeneralDelta(nn.Module):

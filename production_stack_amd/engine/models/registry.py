@@ -53,12 +53,21 @@ def _dogidra_cls():
     return DogidraForCausalLM
 
 
+def _lusolix_cls():
+    from production_stack_amd.engine.models.lusolix import (
+        LusolixForCausalLM,
+    )
+
+    return LusolixForCausalLM
+
+
 MODEL_CLASSES: Dict[str, Callable] = {
     "llama": _llama_cls,
     "nanurax": _nanurax_cls,
     "derusun": _derusun_cls,
     "bipulorn": _bipulorn_cls,
     "dogidra": _dogidra_cls,
+    "lusolix": _lusolix_cls,
 }
 
 
@@ -87,15 +96,22 @@ def _dogidra_config(path: str) -> ModelConfig:
     return dogidra.config_from_dir(path)
 
 
+def _lusolix_config(path: str) -> ModelConfig:
+    from production_stack_amd.engine.models import lusolix
+
+    return lusolix.config_from_dir(path)
+
+
 CONFIG_READERS: Dict[str, Callable[[str], ModelConfig]] = {
     "Nanurax": _nanurax_config,
     "Derusun": _derusun_config,
     "Bipulorn": _bipulorn_config,
     "Dogidra": _dogidra_config,
+    "Lusolix": _lusolix_config,
 }
 
 # families whose layers also run in float32 (the Llama path is bf16-only)
-FP32_FAMILIES = {"nanurax", "derusun", "bipulorn", "dogidra"}
+FP32_FAMILIES = {"nanurax", "derusun", "bipulorn", "dogidra", "lusolix"}
 
 
 def config_from_dir(path: str) -> ModelConfig:

@@ -454,16 +454,26 @@ def _rows(t: torch.Tensor, name: str) -> int:
 
 
 def embed_scale(tokens: torch.Tensor, embed: torch.Tensor,
-                scale: float) -> torch.Tensor:
-    """fp32 residual rows embed[token] * scale."""
-    if not embed.is_cuda:
-        return reference.embed_scale(tokens, embed, scale)
+                scale: float, pos: torch.Tensor = None,
+                positions: torch.Tensor = None) -> torch.Tensor:
+    """fp32 residual rows embed[token] * scale (+ pos[position], a learned
+    position table of embed's dtype, positions int32 [T])."""
     T, W = tokens.shape[0], embed.shape[1]
+    if pos is not None:
+        assert pos.dim() == 2 and pos.shape[1] == W
+        assert pos.dtype == embed.dtype
+        assert positions.dtype == torch.int32 and positions.shape == (T,)
+    if not embed.is_cuda:
+        return reference.embed_scale(tokens, embed, scale, pos, positions)
     assert tokens.dtype == torch.long and tokens.is_contiguous()
     assert embed.is_contiguous()
+    assert pos is None or pos.is_contiguous()
     x = torch.empty((T, W), dtype=torch.float32, device=embed.device)
     _mx().mx_embed_scale(_p(x), _p(tokens), _p(embed),
-                         _f(scale), T, W, _mx_dtype(embed.dtype), _stream())
+                         _f(scale), T, W, _p(pos),
+                         int(pos.shape[0]) if pos is not None else 0,
+                         _p(positions if pos is not None else None),
+                         _mx_dtype(embed.dtype), _stream())
     return x
 
 
@@ -824,14 +834,18 @@ def add_layer_norm_conv32(x32: torch.Tensor, deltas, scales,
                           w32: torch.Tensor, b32: torch.Tensor, eps: float,
                           conv_w: torch.Tensor, state: torch.Tensor,
                           seq_rows: torch.Tensor,
-                          out_dtype: torch.dtype) -> torch.Tensor:
+                          out_dtype: torch.dtype, gate=None,
+                          plain: bool = False):
     """Sublayer boundary with a layer norm and an input convolution (see
     reference.add_layer_norm_conv32): x32 fp32 [T, W] += sum scales[i] *
     deltas[i] in place (up to two deltas [T, W] of one dtype, row-strided
     views allowed), y = layernorm(x32) * w32 + b32, returns y + conv(y) in
     out_dtype, the causal convolution (conv_w fp32 [W, K]) running along
     the segments of seq_rows with state fp32 [slots, K-1, W] (a segment's
-    previous K - 1 rows of y), which is updated. conv_w None: returns y."""
+    previous K - 1 rows of y), which is updated. conv_w None: returns y.
+    gate = (z [T, W] of out_dtype, bias fp32 [W]): the only delta is
+    multiplied by sigmoid(z + bias) as well. plain: returns (y + conv(y),
+    y)."""
     T, W = x32.shape
     assert x32.dtype == torch.float32 and x32.is_contiguous()
     deltas, scales = list(deltas), [float(v) for v in scales]
@@ -846,37 +860,113 @@ def add_layer_norm_conv32(x32: torch.Tensor, deltas, scales,
         assert conv_w.dtype == torch.float32 and conv_w.shape == (W, K)
         assert K >= 1 and state.dtype == torch.float32
         assert state.shape[1:] == (K - 1, W)
+    z = zb = None
+    if gate is not None:
+        z, zb = gate
+        assert len(deltas) == 1 and z.shape == (T, W)
+        assert z.dtype == out_dtype
+        assert zb.dtype == torch.float32 and zb.numel() == W
     if not x32.is_cuda:
         return reference.add_layer_norm_conv32(
             x32, deltas, scales, w32, b32, eps, conv_w, state, seq_rows,
-            out_dtype)
+            out_dtype, gate, plain)
     h = torch.empty((T, W), dtype=out_dtype, device=x32.device)
+    y = h
+    if plain and conv_w is not None:
+        y = torch.empty_like(h)
+    d0 = deltas[0] if deltas else None
+    d1 = deltas[1] if len(deltas) > 1 else None
+    single = 0
     stats = None
     if conv_w is not None:
         _check_seq_rows(seq_rows)
         assert conv_w.is_contiguous() and state.is_contiguous()
-        stats = torch.empty((T, 2), dtype=torch.float32, device=x32.device)
-    d0 = deltas[0] if deltas else None
-    d1 = deltas[1] if len(deltas) > 1 else None
-    _mx().mx_add_layer_norm32(
-        _p(h if conv_w is None else None), _p(x32), _p(d0),
+        # as many segments as rows: every segment is one row, whose
+        # convolution needs the state alone, and one launch does it all
+        single = int(seq_rows.shape[0] == T)
+        if not single:
+            stats = torch.empty((T, 2), dtype=torch.float32,
+                                device=x32.device)
+    rc = _mx().mx_add_layer_norm32(
+        _p(h if conv_w is None or single else None), _p(x32), _p(d0),
         _rows(d0, "delta") if d0 is not None else 0,
         _f(scales[0] if deltas else 0.0), _p(d1),
         _rows(d1, "delta") if d1 is not None else 0,
         _f(scales[1] if d1 is not None else 0.0), _p(w32), _p(b32), _f(eps),
         _p(stats), T, W,
         _mx_dtype(d0.dtype) if d0 is not None else 0, _mx_dtype(out_dtype),
-        _stream())
-    if conv_w is not None:
+        _p(z), _rows(z, "gate") if z is not None else 0, _p(zb),
+        _p(y if single and plain else None), _p(conv_w if single else None),
+        _p(state if single and K > 1 else None),
+        _p(seq_rows if single else None), K if single else 0, _stream())
+    if rc != 0:
+        raise RuntimeError(
+            f"add_layer_norm_conv32: {K} taps are not built (1-32)")
+    if conv_w is not None and not single:
         S = seq_rows.shape[0]
         rc = _mx().mx_norm_conv32(
-            _p(h), _p(x32), _p(stats), _p(w32), _p(b32), _p(conv_w),
-            _p(state), _p(seq_rows), S, W, K, T, _mx_dtype(out_dtype),
-            _stream())
+            _p(h), _p(y if plain else None), _p(x32), _p(stats), _p(w32),
+            _p(b32), _p(conv_w), _p(state), _p(seq_rows), S, W, K, T,
+            _mx_dtype(out_dtype), _stream())
         if rc != 0:
             raise RuntimeError(
                 f"add_layer_norm_conv32: {K} taps are not built (1-32)")
-    return h
+    return (h, y) if plain else h
+
+
+def rms_norm_rows(x: torch.Tensor, w32: torch.Tensor,
+                  eps: float) -> torch.Tensor:
+    """x [T, C] (row-strided view) / its root mean square per row * w32
+    (fp32 [C]), fp32 arithmetic, result of x's dtype."""
+    T, C = x.shape
+    assert w32.dtype == torch.float32 and w32.numel() == C
+    if not x.is_cuda:
+        return reference.rms_norm_rows(x, w32, eps)
+    out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+    _mx().mx_rms_norm_rows(_p(out), _p(x), _rows(x, "x"), _p(w32), _f(eps),
+                           T, C, _mx_dtype(x.dtype), _stream())
+    return out
+
+
+def merge_heads(o: torch.Tensor, gate: torch.Tensor = None,
+                out: torch.Tensor = None) -> torch.Tensor:
+    """Heads side by side: o [H, T, DV] -> [T, H*DV], head h of token t
+    times sigmoid(gate[t, h]) when gate [T, H] (row-strided view) is
+    given."""
+    H, T, DV = o.shape
+    if gate is not None:
+        assert gate.shape == (T, H) and gate.dtype == o.dtype
+    if out is None:
+        out = torch.empty((T, H * DV), dtype=o.dtype, device=o.device)
+    assert out.shape == (T, H * DV) and out.dtype == o.dtype
+    if not o.is_cuda:
+        out.copy_(reference.merge_heads(o, gate))
+        return out
+    assert o.is_contiguous()
+    _mx().mx_merge_heads(
+        _p(out), _rows(out, "out"), _p(o), _p(gate),
+        _rows(gate, "gate") if gate is not None else 0, T, H, DV,
+        _mx_dtype(o.dtype), _stream())
+    return out
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float,
+              out: torch.Tensor = None) -> torch.Tensor:
+    """c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 element by element, N dividing a
+    row by its root mean square; z [T, F] row-strided view, coef fp32 [4]
+    (a device tensor), fp32 arithmetic, result of z's dtype."""
+    T, F = z.shape
+    assert coef.dtype == torch.float32 and coef.shape == (4,)
+    if out is None:
+        out = torch.empty((T, F), dtype=z.dtype, device=z.device)
+    assert out.shape == (T, F) and out.dtype == z.dtype
+    if not z.is_cuda:
+        out.copy_(reference.poly_norm(z, coef, eps))
+        return out
+    _mx().mx_poly_norm(_p(out), _rows(out, "out"), _p(z), _rows(z, "z"),
+                       _p(coef), _f(eps), T, F, _mx_dtype(z.dtype),
+                       _stream())
+    return out
 
 
 def mingru_scan(z: torch.Tensor, u: torch.Tensor, g: torch.Tensor,
@@ -1265,4 +1355,139 @@ def moe_combine(y: torch.Tensor, dense: torch.Tensor, x: torch.Tensor,
         else 0, _p(shared_gate),
         _rows(shared_gate, "shared_gate") if shared_gate is not None else 0,
         T, W, _mx_dtype(y.dtype), _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------
+# routed experts over rows sorted by expert
+# ---------------------------------------------------------------------------
+def _plan_buffers(layers: int, n: int, n_out: int, device):
+    i32 = torch.int32
+    return (torch.empty((layers, n_out + 1), dtype=i32, device=device),
+            torch.empty((layers, n), dtype=i32, device=device),
+            torch.empty((layers, n), dtype=i32, device=device))
+
+
+def expert_plan(sel: torch.Tensor, n_out: int):
+    """sel int64 [T, top], entries in [0, n_out): stable sort of the T * top
+    entries by output. Returns int32 (offs [n_out + 1], rows [T * top] =
+    token of every sorted entry, pos [T * top] = sorted place of every
+    entry)."""
+    T, top = sel.shape
+    assert sel.dtype == torch.long and sel.is_contiguous()
+    if not sel.is_cuda:
+        return reference.expert_plan(sel, n_out)
+    offs, rows, pos = _plan_buffers(1, T * top, n_out, sel.device)
+    rc = _mx().mx_expert_plan(
+        _p(offs), _p(rows), _p(pos), _p(sel), _p(None), _p(None), 1, T, top,
+        n_out, 0, _stream())
+    if rc != 0:
+        raise RuntimeError(f"expert_plan: {n_out} outputs exceed 1024")
+    return offs[0], rows[0], pos[0]
+
+
+def table_plan(tokens: torch.Tensor, tables: torch.Tensor, experts: int):
+    """Plans of several layers whose experts come from tables: tables int32
+    [layers, vocab, top] names the experts of every token id, tokens int64
+    [T]. Returns int32 (offs [layers, experts + 1], rows [layers, T * top],
+    pos [layers, T * top]) as expert_plan would for each layer."""
+    Lm, V, top = tables.shape
+    T = tokens.shape[0]
+    assert tokens.dtype == torch.long and tables.dtype == torch.int32
+    if not tokens.is_cuda:
+        parts = [reference.expert_plan(t[tokens].long(), experts)
+                 for t in tables]
+        return tuple(torch.stack(p) for p in zip(*parts))
+    assert tokens.is_contiguous() and tables.is_contiguous()
+    offs, rows, pos = _plan_buffers(Lm, T * top, experts, tokens.device)
+    rc = _mx().mx_expert_plan(
+        _p(offs), _p(rows), _p(pos), _p(None), _p(tokens), _p(tables), Lm, T,
+        top, experts, V, _stream())
+    if rc != 0:
+        raise RuntimeError(f"table_plan: {experts} experts exceed 1024")
+    return offs, rows, pos
+
+
+def experts_grouped_fits(x: torch.Tensor, w_in: torch.Tensor,
+                         w_out: torch.Tensor) -> bool:
+    """Whether experts_grouped covers these operands: bfloat16, widths that
+    are whole 16-byte vectors."""
+    W, ff = x.shape[1], w_out.shape[2]
+    return (x.dtype == torch.bfloat16 and W % 8 == 0 and ff % 8 == 0
+            and w_in.is_contiguous() and w_out.is_contiguous())
+
+
+def experts_grouped(x: torch.Tensor, w_in: torch.Tensor,
+                    w_out: torch.Tensor, offs: torch.Tensor,
+                    rows: torch.Tensor, act: str, limit: float = 0.0,
+                    gated: bool = True,
+                    row_scale: torch.Tensor = None) -> torch.Tensor:
+    """Every planned entry through its expert in two launches, no host
+    read: y_i = W_out[e] act(W_in[e] x[rows[i]]) for the sorted entries i
+    of expert e (see expert_plan; entries past the last expert are left
+    unwritten). x [T, W]; w_in [E, (2)ff, W] = gate | up rows (up alone
+    when not gated); w_out [E, W, ff]; row_scale fp32 [entries]: the
+    expert reads row_scale[i] * x. Returns [entries, W]. bfloat16, fp32
+    accumulation; the activation reads the unrounded sums."""
+    T, W = x.shape
+    E, n_in, _ = w_in.shape
+    ff = w_out.shape[2]
+    n = rows.numel()
+    assert w_in.shape == (E, (2 if gated else 1) * ff, W)
+    assert w_out.shape == (E, W, ff)
+    assert offs.dtype == torch.int32 and offs.numel() >= E + 1
+    assert rows.dtype == torch.int32 and n > 0
+    if row_scale is not None:
+        assert row_scale.dtype == torch.float32 and row_scale.numel() == n
+    y = torch.empty((n, W), dtype=x.dtype, device=x.device)
+    if not x.is_cuda:
+        reference.experts_grouped(y, x, w_in, w_out, offs, rows, act, limit,
+                                  gated, row_scale)
+        return y
+    if not experts_grouped_fits(x, w_in, w_out):
+        raise ValueError("experts_grouped: bfloat16 with widths that are "
+                         "multiples of 8 only")
+    assert x.is_contiguous() and offs.is_contiguous() and rows.is_contiguous()
+    mid = torch.empty((n, ff), dtype=x.dtype, device=x.device)
+    _mx().mx_experts_in(_p(mid), _p(x), _p(w_in), _p(offs), _p(rows),
+                        _p(row_scale), E, W, ff, int(bool(gated)),
+                        ACT_KINDS[act], _f(limit), _stream())
+    _mx().mx_experts_out(_p(y), _p(mid), _p(w_out), _p(offs), E, W, ff,
+                         _stream())
+    return y
+
+
+def experts_sum(ys: torch.Tensor, pos: torch.Tensor, top: int, weights,
+                weight: float, sel, experts: int, x: torch.Tensor,
+                shared_y: torch.Tensor = None,
+                shared_gate: torch.Tensor = None) -> torch.Tensor:
+    """fp32 [T, W] = sum_k w[t, k] ys[pos[t * top + k]] (in order of k) with
+    w = weights fp32 [T, top], or the number `weight` everywhere; entries
+    whose sel [T, top] (int64, optional) lies at `experts` or beyond stand
+    for the input x itself; the shared expert joins as in moe_combine."""
+    T, W = x.shape
+    assert pos.dtype == torch.int32 and pos.numel() == T * top
+    assert ys.shape == (T * top, W) and ys.dtype == x.dtype
+    if weights is not None:
+        assert weights.dtype == torch.float32 and weights.shape == (T, top)
+    if sel is not None:
+        assert sel.dtype == torch.long and sel.shape == (T, top)
+    if shared_y is not None:
+        assert shared_y.shape == (T, W) and shared_y.dtype == x.dtype
+        if shared_gate is not None:
+            assert shared_gate.shape == (T, 1)
+            assert shared_gate.dtype == x.dtype
+    if not x.is_cuda:
+        return reference.experts_sum(ys, pos, top, weights, weight, sel,
+                                     experts, x, shared_y, shared_gate)
+    for t in (ys, pos, weights, sel):
+        assert t is None or t.is_contiguous()
+    out = torch.empty((T, W), dtype=torch.float32, device=x.device)
+    _mx().mx_experts_sum(
+        _p(out), _p(ys), _p(pos), int(top), _p(weights), _f(weight),
+        _p(sel), int(experts), _p(x), _rows(x, "x"), _p(shared_y),
+        _rows(shared_y, "shared_y") if shared_y is not None else 0,
+        _p(shared_gate),
+        _rows(shared_gate, "shared_gate") if shared_gate is not None else 0,
+        T, W, _mx_dtype(x.dtype), _stream())
     return out

@@ -207,9 +207,13 @@ def lora_bgmv(out, x, A, B, scale, idx, col_off):
 # ---------------------------------------------------------------------------
 # fp32-residual stack ops (hybrid recurrent/attention models)
 # ---------------------------------------------------------------------------
-def embed_scale(tokens, embed, scale: float) -> torch.Tensor:
-    """fp32 residual stream rows: embed[token] * scale."""
-    return embed[tokens].float() * scale
+def embed_scale(tokens, embed, scale: float, pos=None,
+                positions=None) -> torch.Tensor:
+    """fp32 residual stream rows: embed[token] * scale (+ pos[position])."""
+    x = embed[tokens].float() * scale
+    if pos is not None:
+        x = x + pos[positions.long()].float()
+    return x
 
 
 def add_rms_norm32(x32, deltas, w32, eps: float, out_dtype, groups: int = 1,
@@ -489,7 +493,8 @@ def pool_append(k_cache, v_cache, kp_cache, vp_cache, block_tables,
 
 
 def add_layer_norm_conv32(x32, deltas, scales, w32, b32, eps: float,
-                          conv_w, state, seq_rows, out_dtype):
+                          conv_w, state, seq_rows, out_dtype, gate=None,
+                          plain: bool = False):
     """Sublayer boundary of a stack with layer norms and input
     convolutions: x32 += sum_i scales[i] * deltas[i] (fp32, in place), y =
     (x32 - mean) / sqrt(var + eps) * w32 + b32 per row, and the returned
@@ -497,18 +502,22 @@ def add_layer_norm_conv32(x32, deltas, scales, w32, b32, eps: float,
     y_(t - K + 1 + j) along each segment of seq_rows with the segment's
     previous K - 1 rows of y taken from state fp32 [slots, K-1, W] (zeros
     for a segment that starts at position 0); state receives the last K - 1
-    rows. conv_w None: h = y."""
+    rows. conv_w None: h = y. gate = (z, bias): the only delta times
+    sigmoid(z + bias) joins. plain: returns (h, y)."""
     if deltas:
         acc = None
         for d, sc in zip(deltas, scales):
             term = d.float() * sc
+            if gate is not None:
+                term = term * torch.sigmoid(gate[0].float() + gate[1])
             acc = term if acc is None else acc + term
         x32.add_(acc)
     mu = x32.mean(-1, keepdim=True)
     var = (x32 - mu).pow(2).mean(-1, keepdim=True)
     y = (x32 - mu) * torch.rsqrt(var + eps) * w32 + b32
     if conv_w is None:
-        return y.to(out_dtype)
+        h = y.to(out_dtype)
+        return (h, h) if plain else h
     T, W = y.shape
     K = conv_w.shape[1]
     h = torch.empty_like(y)
@@ -521,7 +530,37 @@ def add_layer_norm_conv32(x32, deltas, scales, w32, b32, eps: float,
         h[t0:t0 + n] = acc
         if K > 1:
             state[slot] = ext[n:]
-    return h.to(out_dtype)
+    return (h.to(out_dtype), y.to(out_dtype)) if plain else h.to(out_dtype)
+
+
+def rms_norm_rows(x, w32, eps: float):
+    """x [T, C] / its root mean square per row * w32, in x's dtype."""
+    xf = x.float()
+    return (xf * torch.rsqrt(xf.pow(2).mean(-1, keepdim=True) + eps)
+            * w32).to(x.dtype)
+
+
+def merge_heads(o, gate=None):
+    """o [H, T, DV] -> [T, H*DV], head h of token t times
+    sigmoid(gate[t, h])."""
+    H, T, DV = o.shape
+    y = o.transpose(0, 1).float()
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float()).unsqueeze(-1)
+    return y.reshape(T, H * DV).to(o.dtype)
+
+
+def poly_norm(z, coef, eps: float):
+    """c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 in fp32, N: over the row's root
+    mean square."""
+    y = None
+    zf = z.float()
+    p = zf
+    for k in range(3):
+        n = coef[k] * p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)
+        y = n if y is None else y + n
+        p = p * zf
+    return (y + coef[3]).to(z.dtype)
 
 
 def mingru_scan(z, u, g, zb, ub, state, seq_rows, out_dtype):
@@ -806,6 +845,59 @@ def moe_combine(y, dense, x, experts: int, shared_y=None, shared_gate=None):
     out = torch.einsum("te,etw->tw", dense[:, :experts], y.float())
     if dense.shape[1] > experts:
         out = out + dense[:, experts:].sum(-1, keepdim=True) * x.float()
+    if shared_y is not None and shared_gate is not None:
+        out = out + torch.sigmoid(shared_gate.float()) * shared_y.float()
+    elif shared_y is not None:
+        out = out + shared_y.float()
+    return out
+
+
+def expert_plan(sel, n_out: int):
+    """Stable sort of the entries of sel [T, top] by output: int32 (offs
+    [n_out + 1], rows = token of every sorted entry, pos = sorted place of
+    every entry)."""
+    T, top = sel.shape
+    flat = sel.reshape(-1)
+    order = torch.argsort(flat, stable=True)
+    pos = torch.empty(T * top, dtype=torch.int32)
+    pos[order] = torch.arange(T * top, dtype=torch.int32)
+    offs = torch.zeros(n_out + 1, dtype=torch.int32)
+    offs[1:] = torch.cumsum(torch.bincount(flat, minlength=n_out), 0)
+    rows = torch.div(order, top, rounding_mode="floor").int()
+    return offs, rows, pos
+
+
+def experts_grouped(y, x, w_in, w_out, offs, rows, act: str, limit: float,
+                    gated: bool, row_scale=None) -> None:
+    """y[i] = W_out[e] act(W_in[e] (row_scale[i] x[rows[i]])) for the sorted
+    entries i of expert e; the activation reads unrounded fp32 sums."""
+    ff = w_out.shape[2]
+    o = offs.tolist()
+    for e in range(w_in.shape[0]):
+        a, b = o[e], o[e + 1]
+        if a == b:
+            continue
+        g = x[rows[a:b].long()].float() @ w_in[e].float().t()
+        if row_scale is not None:
+            g = g * row_scale[a:b, None]
+        h = (gated_act(g[:, :ff], g[:, ff:], act, limit, x.dtype) if gated
+             else gated_act(g, None, act, limit, x.dtype))
+        y[a:b] = (h.float() @ w_out[e].float().t()).to(y.dtype)
+
+
+def experts_sum(ys, pos, top: int, weights, weight: float, sel,
+                experts: int, x, shared_y=None, shared_gate=None):
+    """fp32 [T, W]: weighted sum over the top entries of every token (input
+    itself where sel >= experts), plus the (gated) shared expert."""
+    T, W = x.shape
+    y = ys[pos.long()].view(T, top, W).float()
+    if sel is not None:
+        y = torch.where((sel >= experts).unsqueeze(-1),
+                        x.float().unsqueeze(1), y)
+    out = torch.zeros(T, W)
+    for k in range(top):
+        w = weights[:, k:k + 1] if weights is not None else weight
+        out = out + w * y[:, k]
     if shared_y is not None and shared_gate is not None:
         out = out + torch.sigmoid(shared_gate.float()) * shared_y.float()
     elif shared_y is not None:
