@@ -178,6 +178,10 @@ PS_DEV float mg_act(int kind, float g, float u, bool gated, float limit) {
 
 #define MG_ACT_NONE (-1)
 
+PS_DEV float mg_round(float v) {
+  return ps_bf16_to_f32(ps_f32_to_bf16(v));
+}
+
 // Four 16-row weight tiles (row pointers wp, one per tile and lane) times RT
 // 16-row tiles of inputs (row pointers xp): this wave's share of K.
 template <int RT>
@@ -300,9 +304,11 @@ PS_DEV void mg_rows(unsigned short* __restrict__ out,
           float y[4];
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            y[i] = sc * s[p][i];
+            // rounded here as a GEMM of its own would round its result, so
+            // small and large batches agree
+            y[i] = mg_round(sc * s[p][i]);
             if (PAIR)
-              y[i] = mg_act(act, y[i], sc * s[1][i], true, limit);
+              y[i] = mg_act(act, y[i], mg_round(sc * s[1][i]), true, limit);
             else if (act != MG_ACT_NONE)
               y[i] = mg_act(act, y[i], 1.f, false, limit);
           }

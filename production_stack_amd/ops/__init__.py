@@ -1428,7 +1428,8 @@ def experts_grouped(x: torch.Tensor, w_in: torch.Tensor,
     unwritten). x [T, W]; w_in [E, (2)ff, W] = gate | up rows (up alone
     when not gated); w_out [E, W, ff]; row_scale fp32 [entries]: the
     expert reads row_scale[i] * x. Returns [entries, W]. bfloat16, fp32
-    accumulation; the activation reads the unrounded sums."""
+    accumulation; rounded at the same places as one GEMM pair per expert
+    with the activation between them."""
     T, W = x.shape
     E, n_in, _ = w_in.shape
     ff = w_out.shape[2]

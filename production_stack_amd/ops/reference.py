@@ -870,7 +870,8 @@ def expert_plan(sel, n_out: int):
 def experts_grouped(y, x, w_in, w_out, offs, rows, act: str, limit: float,
                     gated: bool, row_scale=None) -> None:
     """y[i] = W_out[e] act(W_in[e] (row_scale[i] x[rows[i]])) for the sorted
-    entries i of expert e; the activation reads unrounded fp32 sums."""
+    entries i of expert e; the activation reads the projection rounded to
+    the element type, as it does between separate GEMMs."""
     ff = w_out.shape[2]
     o = offs.tolist()
     for e in range(w_in.shape[0]):
@@ -880,6 +881,7 @@ def experts_grouped(y, x, w_in, w_out, offs, rows, act: str, limit: float,
         g = x[rows[a:b].long()].float() @ w_in[e].float().t()
         if row_scale is not None:
             g = g * row_scale[a:b, None]
+        g = g.to(x.dtype)
         h = (gated_act(g[:, :ff], g[:, ff:], act, limit, x.dtype) if gated
              else gated_act(g, None, act, limit, x.dtype))
         y[a:b] = (h.float() @ w_out[e].float().t()).to(y.dtype)
