@@ -123,6 +123,7 @@ COMPARE_PAIRS = {
                  ("bipulorn-8b", "nanurax-8b")],
     "dogidra": [("dogidra-1b", "bipulorn-1b"),
                 ("dogidra-8b", "bipulorn-8b")],
+    "lusolix": [("lusolix-1b", "dogidra-1b"), ("lusolix-8b", "dogidra-8b")],
 }
 
 

@@ -10,6 +10,8 @@
 //                    latent a query passes);
 //   merge_heads      per-head outputs side by side, each head times the
 //                    sigmoid of its gate;
+//   latent_gather    rows of a paged cache side by side (the rows a step's
+//                    prompt portions see, for expansion);
 //   pool_append      mean key/value of every block of positions a step
 //                    completes, into the pooled caches;
 //   short_conv_silu  causal per-channel convolution over time + silu with
@@ -191,8 +193,7 @@ PS_DEV void mx_turn(float u, float w, const float* cs, float* ou, float* ow) {
 
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prep_kernel(
-    T* __restrict__ qf, const T* __restrict__ qlat, const T* __restrict__ q,
-    int ldq, const T* __restrict__ dkv, int lddkv,
+    T* qf, const T* __restrict__ qlat, const T* q, int ldq, const T* __restrict__ dkv, int lddkv,
     const float* __restrict__ normw, float eps,
     const float* __restrict__ cos_sin, int table_rows, int rot_dims,
     const int* __restrict__ positions, T* __restrict__ cache,
@@ -225,6 +226,19 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     }
     if ((R & 1) && threadIdx.x == 0)
       crow[L + R - 1] = row[L + R - 1];
+  }
+  if (qlat == nullptr) {
+    // queries stay as they are, their rotary parts turn in place (qf is q);
+    // a thread owns both entries of a pair
+    for (int c = threadIdx.x; c < H * (rot_dims / 2); c += blockDim.x) {
+      const int h = c / (rot_dims / 2), i = c - h * (rot_dims / 2);
+      T* p = qf + (size_t)t * ldq + h * (D + R) + D + 2 * i;
+      float u, w;
+      mx_turn(MxElem<T>::ld(p), MxElem<T>::ld(p + 1), cs + 2 * i, &u, &w);
+      MxElem<T>::st(p, u);
+      MxElem<T>::st(p + 1, w);
+    }
+    return;
   }
   // queries: per head [latent-space part | turned rotary part]
   const int QW = L + R;
@@ -266,18 +280,18 @@ __global__ __launch_bounds__(256) void rms_norm_rows_kernel(
     MxElem<T>::st(yr + c, MxElem<T>::ld(xr + c) * inv * w[c]);
 }
 
-// out[t, h*DV + d] = o[h][t][d] * sigmoid(gate[t, h]) (gate nullptr: the
-// plain copy). Grid (column chunks, tokens); a thread takes V consecutive
+// out[t, h*DV + d] = o[h*hs + t*rs + d] * sigmoid(gate[t, h]) (gate nullptr:
+// the plain copy). out may be o itself where both lie the same way. Grid (column chunks, tokens); a thread takes V consecutive
 // entries of one head (V divides DV).
 template <typename T, int V>
 __global__ __launch_bounds__(256) void merge_heads_kernel(
-    T* __restrict__ out, int ldo, const T* __restrict__ o,
-    const T* __restrict__ gate, int ldg, int T_, int H, int DV) {
+    T* out, int ldo, const T* o, int64_t hs, int64_t rs,
+    const T* __restrict__ gate, int ldg, int H, int DV) {
   const int t = blockIdx.y;
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * V;
   if (c >= H * DV) return;
   const int h = c / DV, d = c - h * DV;
-  const T* src = o + ((size_t)h * T_ + t) * DV + d;
+  const T* src = o + h * hs + t * rs + d;
   T* dst = out + (size_t)t * ldo + c;
   const float g = gate != nullptr
                       ? mx_sigmoid(MxElem<T>::ld(gate + (size_t)t * ldg + h))
@@ -290,6 +304,23 @@ __global__ __launch_bounds__(256) void merge_heads_kernel(
 #pragma unroll
   for (int i = 0; i < V; ++i) MxElem<T>::st(&r.e[i], MxElem<T>::ld(&v.e[i]) * g);
   *(Vec*)dst = r;
+}
+
+// One wave per row: segment blockIdx.y's row r comes from position p0 + r of
+// its sequence. U: copy unit.
+template <typename U>
+__global__ __launch_bounds__(256) void latent_gather_kernel(
+    U* __restrict__ out, const U* __restrict__ cache,
+    const int* __restrict__ block_tables, int max_blocks,
+    const int* __restrict__ segments, int BS, int units) {
+  const int* sg = segments + 3 * blockIdx.y;
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (r >= sg[1]) return;
+  const int p = sg[2] + r;
+  const int blk = block_tables[(size_t)blockIdx.y * max_blocks + p / BS];
+  const U* src = cache + ((int64_t)blk * BS + p % BS) * units;
+  U* dst = out + ((int64_t)sg[0] + r) * units;
+  for (int c = threadIdx.x & 63; c < units; c += 64) dst[c] = src[c];
 }
 
 // Thread = channel, workgroup = (channel tile, segment, chunk of CONV_CH
@@ -426,25 +457,46 @@ void mx_rms_norm_rows(void* y, const void* x, int ldx, const void* w,
   })
 }
 
-void mx_merge_heads(void* out, int ldo, const void* o, const void* gate,
-                    int ldg, int T_, int H, int DV, int dtype,
-                    void* stream) {
+void mx_merge_heads(void* out, int ldo, const void* o, int hs, int rs,
+                    const void* gate, int ldg, int T_, int H, int DV,
+                    int dtype, void* stream) {
   if (T_ <= 0 || H * DV <= 0) return;
   const bool aligned = (((size_t)out | (size_t)o) & 15) == 0;
   MX_DISPATCH_DTYPE(dtype, {
     constexpr int V = 16 / sizeof(T);
-    if (aligned && DV % V == 0 && ldo % V == 0) {
+    if (aligned && DV % V == 0 && ldo % V == 0 && hs % V == 0 &&
+        rs % V == 0) {
       hipLaunchKernelGGL((merge_heads_kernel<T, V>),
                          dim3((H * DV / V + 255) / 256, T_), dim3(256), 0,
                          (hipStream_t)stream, (T*)out, ldo, (const T*)o,
-                         (const T*)gate, ldg, T_, H, DV);
+                         (int64_t)hs, (int64_t)rs, (const T*)gate, ldg, H,
+                         DV);
     } else {
       hipLaunchKernelGGL((merge_heads_kernel<T, 1>),
                          dim3((H * DV + 255) / 256, T_), dim3(256), 0,
                          (hipStream_t)stream, (T*)out, ldo, (const T*)o,
-                         (const T*)gate, ldg, T_, H, DV);
+                         (int64_t)hs, (int64_t)rs, (const T*)gate, ldg, H,
+                         DV);
     }
   })
+}
+
+void mx_latent_gather(void* out, const void* cache, const void* block_tables,
+                      int max_blocks, const void* segments, int S_,
+                      int longest, int BS, int D, int dtype, void* stream) {
+  if (S_ <= 0 || longest <= 0) return;
+  const int bytes = D * (dtype == MX_BF16 ? 2 : 4);
+  dim3 grid((longest + 3) / 4, S_);
+#define LG_GO(U)                                                            \
+  hipLaunchKernelGGL((latent_gather_kernel<U>), grid, dim3(256), 0,         \
+                     (hipStream_t)stream, (U*)out, (const U*)cache,         \
+                     (const int*)block_tables, max_blocks,                  \
+                     (const int*)segments, BS, bytes / (int)sizeof(U))
+  if (bytes % 16 == 0 && (((size_t)out | (size_t)cache) & 15) == 0)
+    LG_GO(uint4);
+  else
+    LG_GO(unsigned short);
+#undef LG_GO
 }
 
 #define CONV_CASE(KK)                                                        \

@@ -464,6 +464,7 @@ class ModelRunner:
                     dev, non_blocking=True),
                 seq_rows=torch.from_numpy(rows_np).to(
                     dev, non_blocking=True),
+                seq_rows_host=rows_np.tolist(),
             )
 
         meta = BatchMeta(

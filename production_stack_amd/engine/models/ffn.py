@@ -322,6 +322,7 @@ class SparseMoE(nn.Module):
         act = self._act(gemm_policy.linear(xe, self.experts_gate_up[e]))
         return gemm_policy.linear(act, self.experts_down[e])
 
+    @torch.no_grad()
     def _sorted_experts(self, x: torch.Tensor,
                         plan: ExpertPlan) -> torch.Tensor:
         """Sorted entries' outputs [T * top, W] (identity entries, which

@@ -55,6 +55,8 @@ class BatchMeta:
         token_seq: Optional[torch.Tensor] = None,  # [T] int32 row of above
         # [S, 4] int32: first batch row, rows, first position, state slot
         seq_rows: Optional[torch.Tensor] = None,
+        # the same rows on the host (None inside captured graphs)
+        seq_rows_host: Optional[list] = None,
     ) -> None:
         self.positions = positions
         self.slot_mapping = slot_mapping
@@ -73,6 +75,7 @@ class BatchMeta:
         self.block_tables = block_tables
         self.token_seq = token_seq
         self.seq_rows = seq_rows
+        self.seq_rows_host = seq_rows_host
 
 
 def build_cos_sin_cache(

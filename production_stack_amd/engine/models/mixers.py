@@ -214,9 +214,19 @@ class LatentAttention(nn.Module):
     kv_rank + rot_dim numbers per token are cached. `window` limits the
     visible keys to the trailing ones; with `q_rank` the queries pass a
     normalised latent of their own; with `head_gate` every head's output is
-    multiplied by the sigmoid of one projected number."""
+    multiplied by the sigmoid of one projected number.
+
+    Prompt portions that are not tiny against the keys they see take the
+    unfolded form instead: the visible cached rows are gathered and expanded
+    once per step (two GEMMs), and attention runs over dim + rot_dim / vdim
+    entries per head, a third or less of the folded form's products."""
 
     kind = "latent_attention"
+
+    # expand when the visible keys are at most this many times the portion's
+    # tokens, within this many bytes of expanded keys and values
+    EXPAND_RATIO = 16
+    EXPAND_BYTES = 4 << 30
 
     def __init__(self, width: int, spec: MixerSpec, dtype: torch.dtype,
                  eps: float, max_pos: int) -> None:
@@ -252,6 +262,12 @@ class LatentAttention(nn.Module):
             torch.empty(width, H * DV, dtype=dtype))
         self.scale = spec.scale or 1.0 / math.sqrt(D + R)
         self._cos_sin = None
+        self._unfolded = None
+
+    def _apply(self, fn, *a, **kw):
+        # the unfolded weights are plain tensors rebuilt after a move
+        self._unfolded = None
+        return super()._apply(fn, *a, **kw)
 
     def in_params(self):
         return [self.in_proj]
@@ -264,6 +280,63 @@ class LatentAttention(nn.Module):
                 f"value up-projection: checkpoint shape {tuple(t.shape)} != "
                 f"{(H * DV, L)}")
         self.uv.data.copy_(t.to(self.uv.dtype).view(H, DV, L).transpose(1, 2))
+        self._unfolded = None
+
+    def unfolded(self):
+        """(key weight [H*(dim+rot_dim), L+rot_dim], value weight [H*vdim,
+        L]) over cached rows [latent | rotary part]: the key weight's rotary
+        rows pick the shared part as it is, so one GEMM lays down whole
+        keys."""
+        w = self._unfolded
+        if w is None:
+            H, D, R, L, DV = self.H, self.D, self.R, self.L, self.DV
+            k = torch.zeros((H, D + R, L + R), dtype=self.uk.dtype,
+                            device=self.uk.device)
+            k[:, :D, :L] = self.uk.data
+            k[:, D:, L:] = torch.eye(R, dtype=k.dtype, device=k.device)
+            v = self.uv.data.transpose(1, 2).reshape(H * DV, L).contiguous()
+            w = self._unfolded = (k.view(H * (D + R), L + R), v)
+        return w
+
+    def _expansion(self, meta, npt: int, shared: dict):
+        """The step's plan of expanded prompt portions (None: folded form):
+        (segment table int32 [S, 3] = first expanded row, rows, first
+        position; rows in all, longest segment, row table [S, longest],
+        positions counted from the segments' first rows). Layers with one
+        window share it."""
+        host = getattr(meta, "seq_rows_host", None)
+        if host is None or npt == 0:
+            return None
+        win = self.spec.window
+        key = ("latent_expansion", win)
+        if key not in shared:
+            segs, at, rows = [], 0, 0
+            for _, n, p0, _ in host:
+                if rows >= npt:
+                    break
+                lo = max(0, p0 - win + 1) if win else 0
+                segs.append((at, p0 + n - lo, lo))
+                at += p0 + n - lo
+                rows += n
+            plan = None
+            if rows == npt and at <= self.EXPAND_RATIO * npt:
+                dev = meta.positions.device
+                seg = torch.tensor(segs, dtype=torch.int32).to(
+                    dev, non_blocking=True)
+                longest = max(s[1] for s in segs)
+                table = (seg[:, :1] + torch.arange(
+                    longest, dtype=torch.int32, device=dev)).clamp_(
+                        max=at - 1)
+                pos = meta.positions[:npt] - seg[:, 2][
+                    meta.token_seq[:npt].long()]
+                plan = (seg, at, longest, table, pos)
+            shared[key] = plan
+        plan = shared[key]
+        if plan is not None:
+            size = plan[1] * self.H * (self.D + self.R + self.DV)
+            if size * self.uk.element_size() > self.EXPAND_BYTES:
+                return None
+        return plan
 
     @property
     def out_in(self) -> int:
@@ -292,27 +365,54 @@ class LatentAttention(nn.Module):
         if self.q_rank:
             q = gemm_policy.linear(
                 ops.rms_norm_rows(q, self.q_norm, self.eps), self.uq)
+        o = out if out is not None else torch.empty(
+            (T, H * DV), dtype=h.dtype, device=h.device)
+        gate = proj[:, self.q_rows + L + R:] if sp.head_gate else None
+        cs, rd = self.cos_sin(h.device), sp.rot_dims or R
+        npt = min(getattr(meta, "num_prefill_tokens", T) or 0, T)
+        plan = self._expansion(meta, npt, shared)
+        n = npt if plan is not None else 0
+        if n:
+            qn = q[:n]
+            ops.latent_prep(None, qn, dkv[:n], self.latent_norm, self.eps,
+                            cs, meta.positions[:n], cache,
+                            meta.slot_mapping[:n], H, D, R, rd)
+            seg, total, longest, table, pos = plan
+            rows = ops.latent_gather(cache, meta.block_tables, seg, total,
+                                     longest)
+            wk, wv = self.unfolded()
+            k = gemm_policy.linear(rows, wk)
+            v = gemm_policy.linear(rows[:, :L], wv)
+            ops.talk_attention(
+                qn, k.view(total, H, 1, D + R), v.view(total, H, 1, DV),
+                table, meta.token_seq[:n], pos, self.scale, H,
+                window=sp.window, sink=sp.sink, out=o[:n],
+                softcap=sp.softcap, sink_vals=self.sink_vals)
+            if gate is not None:
+                ops.gate_heads(o[:n], gate[:n])
+        if n == T:
+            return o
         # position-free query part into the latent space: [H, T, L]
-        q_lat = torch.bmm(q.view(T, H, D + R)[:, :, :D].transpose(0, 1),
+        q, m = q[n:], T - n
+        q_lat = torch.bmm(q.view(m, H, D + R)[:, :, :D].transpose(0, 1),
                           self.uk)
         qf = ops.latent_prep(
-            q_lat, q, dkv, self.latent_norm, self.eps,
-            self.cos_sin(h.device), meta.positions, cache,
-            meta.slot_mapping, H, D, R, sp.rot_dims or R)
-        o_lat = torch.empty((T, H * L), dtype=h.dtype, device=h.device)
-        npt = min(getattr(meta, "num_prefill_tokens", T) or 0, T)
-        for a, b, variant in ((0, npt, 0), (npt, T, 3)):
+            q_lat, q, dkv[n:], self.latent_norm, self.eps, cs,
+            meta.positions[n:], cache, meta.slot_mapping[n:], H, D, R, rd)
+        o_lat = torch.empty((m, H * L), dtype=h.dtype, device=h.device)
+        for a, b, variant in ((n, npt, 0), (npt, T, 3)):
             if b > a:
                 ops.talk_attention(
-                    qf[a:b], cache, cache, meta.block_tables,
+                    qf[a - n:b - n], cache, cache, meta.block_tables,
                     meta.token_seq[a:b], meta.positions[a:b], self.scale, H,
-                    window=sp.window, sink=sp.sink, out=o_lat[a:b],
+                    window=sp.window, sink=sp.sink, out=o_lat[a - n:b - n],
                     variant=variant, softcap=sp.softcap,
                     sink_vals=self.sink_vals, vdim=L)
         # expand the attended latents per head: [H, T, L] x [H, L, DV]
-        o = torch.bmm(o_lat.view(T, H, L).transpose(0, 1), self.uv)
-        gate = proj[:, self.q_rows + L + R:] if sp.head_gate else None
-        return ops.merge_heads(o, gate, out=out)
+        ops.merge_heads(
+            torch.bmm(o_lat.view(m, H, L).transpose(0, 1), self.uv),
+            gate[n:] if gate is not None else None, out=o[n:])
+        return o
 
 
 class GeneralDelta(nn.Module):

@@ -944,9 +944,48 @@ def merge_heads(o: torch.Tensor, gate: torch.Tensor = None,
         return out
     assert o.is_contiguous()
     _mx().mx_merge_heads(
-        _p(out), _rows(out, "out"), _p(o), _p(gate),
+        _p(out), _rows(out, "out"), _p(o), T * DV, DV, _p(gate),
         _rows(gate, "gate") if gate is not None else 0, T, H, DV,
         _mx_dtype(o.dtype), _stream())
+    return out
+
+
+def gate_heads(o: torch.Tensor, gate: torch.Tensor) -> None:
+    """o [T, H*DV] (row-strided view), in place: head h of token t times
+    sigmoid(gate[t, h]), gate [T, H] (row-strided view)."""
+    T, H = gate.shape
+    DV = o.shape[1] // H
+    assert o.shape == (T, H * DV) and gate.dtype == o.dtype
+    if not o.is_cuda:
+        y = reference.merge_heads(o.view(T, H, DV).transpose(0, 1), gate)
+        o.copy_(y)
+        return
+    ld = _rows(o, "o")
+    _mx().mx_merge_heads(_p(o), ld, _p(o), DV, ld, _p(gate),
+                         _rows(gate, "gate"), T, H, DV, _mx_dtype(o.dtype),
+                         _stream())
+
+
+def latent_gather(cache: torch.Tensor, block_tables: torch.Tensor,
+                  segments: torch.Tensor, total: int,
+                  longest: int) -> torch.Tensor:
+    """Rows of a paged cache [NB, 1, BS, D] side by side: segments int32
+    [S, 3] = (first output row, rows, first position) of the sequences whose
+    block tables are block_tables[:S]; together they fill `total` rows, the
+    longest has `longest`. Returns [total, D]."""
+    NB, one, BS, D = cache.shape
+    S = segments.shape[0]
+    assert one == 1 and block_tables.dtype == torch.int32
+    assert block_tables.dim() == 2 and block_tables.shape[0] >= S
+    assert segments.dtype == torch.int32 and segments.shape[1] == 3
+    if not cache.is_cuda:
+        return reference.latent_gather(cache, block_tables, segments, total)
+    assert cache.is_contiguous() and block_tables.is_contiguous()
+    assert segments.is_contiguous()
+    out = torch.empty((total, D), dtype=cache.dtype, device=cache.device)
+    _mx().mx_latent_gather(
+        _p(out), _p(cache), _p(block_tables), block_tables.shape[1],
+        _p(segments), S, longest, BS, D, _mx_dtype(cache.dtype), _stream())
     return out
 
 
@@ -1012,12 +1051,16 @@ def latent_prep(q_lat: torch.Tensor, q: torch.Tensor, dkv: torch.Tensor,
     """Inputs of latent attention (see reference.latent_prep): normalises
     the latent, turns the shared key part and the queries' rotated parts
     by their positions, appends [latent | key part] to the paged cache
-    [NB, 1, BS, L+rot_dim] and returns the queries [T, H*(L+rot_dim)]."""
+    [NB, 1, BS, L+rot_dim] and returns the queries [T, H*(L+rot_dim)].
+    q_lat None: the queries stay [position-free | rotated] per head; their
+    rotated parts turn in place in q, which is returned."""
     H = heads
     T = q.shape[0]
     L = dkv.shape[1] - rot_dim
     assert q.shape == (T, H * (dim + rot_dim))
-    assert q_lat.shape == (H, T, L) and q_lat.is_contiguous()
+    if q_lat is not None:
+        assert q_lat.shape == (H, T, L) and q_lat.is_contiguous()
+        assert q_lat.dtype == q.dtype
     assert cache.shape[1] == 1 and cache.shape[3] == L + rot_dim
     assert rot_dims % 2 == 0 and rot_dims <= rot_dim
     assert cos_sin.dtype == torch.float32
@@ -1028,10 +1071,13 @@ def latent_prep(q_lat: torch.Tensor, q: torch.Tensor, dkv: torch.Tensor,
         return reference.latent_prep(
             q_lat, q, dkv, norm_w, eps, cos_sin, positions, cache,
             slot_mapping, H, dim, rot_dim, rot_dims, q.dtype)
-    assert q.dtype == dkv.dtype == q_lat.dtype == cache.dtype
+    assert q.dtype == dkv.dtype == cache.dtype
     assert norm_w.dtype == torch.float32 and norm_w.numel() == L
     assert cache.is_contiguous() and cos_sin.is_contiguous()
-    out = torch.empty((T, H * (L + rot_dim)), dtype=q.dtype, device=q.device)
+    out = q
+    if q_lat is not None:
+        out = torch.empty((T, H * (L + rot_dim)), dtype=q.dtype,
+                          device=q.device)
     _mx().mx_latent_prep(
         _p(out), _p(q_lat), _p(q), _rows(q, "q"), _p(dkv),
         _rows(dkv, "dkv"), _p(norm_w), _f(eps), _p(cos_sin),

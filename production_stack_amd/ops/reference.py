@@ -594,7 +594,8 @@ def latent_prep(q_lat, q, dkv, norm_w, eps: float, cos_sin, positions,
     [T, L+rot_dim]: the first L entries are RMS-normalised (norm_w) into
     the latent, the rest is the shared rotated key part. The cache
     [NB, 1, BS, L+rot_dim] receives [latent | turned key part]; returns
-    the queries [T, H*(L+rot_dim)] = per head [q_lat | turned part]."""
+    the queries [T, H*(L+rot_dim)] = per head [q_lat | turned part]; q_lat
+    None: q itself, its rotated parts turned in place."""
     H = heads
     T = q.shape[0]
     L = dkv.shape[1] - rot_dim
@@ -608,8 +609,22 @@ def latent_prep(q_lat, q, dkv, norm_w, eps: float, cos_sin, positions,
         row.to(cache.dtype)
     qr = q.float().view(T, H, dim + rot_dim)[..., dim:]
     qr = _rotate(qr, cs[:, None], rot_dims)
+    if q_lat is None:
+        q.view(T, H, dim + rot_dim)[..., dim:] = qr.to(q.dtype)
+        return q
     full = torch.cat([q_lat.float().transpose(0, 1), qr], dim=-1)
     return full.reshape(T, H * (L + rot_dim)).to(out_dtype)
+
+
+def latent_gather(cache, block_tables, segments, total: int):
+    """[total, D]: cached rows of the segments (first output row, rows,
+    first position), segment i through block_tables[i]."""
+    bs = cache.shape[2]
+    out = torch.empty((total, cache.shape[3]), dtype=cache.dtype)
+    for i, (r0, n, p0) in enumerate(segments.tolist()):
+        p = torch.arange(p0, p0 + n)
+        out[r0:r0 + n] = cache[block_tables[i, p // bs].long(), 0, p % bs]
+    return out
 
 
 def short_conv_silu(x, w, state, seq_rows, out_dtype, bias=None):

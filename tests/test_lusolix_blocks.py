@@ -1,0 +1,502 @@
+"""Each Lusolix mechanism alone: the engine's ops and modules (in portions,
+through scattered and previously used pages and slots) against the float64
+oracle in tests/oracle_lusolix.py, and, marked gpu, the HIP kernels against
+the reference ops."""
+
+import pytest
+import torch
+
+import oracle_lusolix as O
+from lusolix_util import (TOL, dense, make_cfg, make_weights, mixer, moe,
+                          rel_err, save_checkpoint)
+from production_stack_amd import ops
+from production_stack_amd.engine.models import registry
+from production_stack_amd.engine.models.ffn import TablePlans
+from production_stack_amd.engine.models.llama import BatchMeta
+from production_stack_amd.ops import reference as R
+
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+DTYPES = ["float32", "bfloat16"]
+TD = {"float32": torch.float32, "bfloat16": torch.bfloat16}
+F64 = torch.float64
+
+pytestmark = pytest.mark.filterwarnings("ignore::UserWarning")
+
+
+def rnd(shape, seed, scale=1.0, dtype=torch.float32):
+    g = torch.Generator().manual_seed(seed)
+    return (torch.randn(*shape, generator=g) * scale).to(dtype)
+
+
+def relerr(got, want):
+    got, want = got.detach().cpu().to(F64), want.detach().cpu().to(F64)
+    return float((got - want).norm() / want.norm().clamp_min(1e-12))
+
+
+def seq_rows(parts, device="cpu"):
+    """parts: [(rows, first position, slot)]."""
+    rows, r0 = [], 0
+    for n, p0, slot in parts:
+        rows.append([r0, n, p0, slot])
+        r0 += n
+    return torch.tensor(rows, dtype=torch.int32, device=device)
+
+
+def load_layer(layer, mlp, W, width, dtype, device, taps=3):
+    """A one-layer model read through the registry, as the engine reads
+    it."""
+    import tempfile
+
+    cfg = make_cfg([(layer, mlp)], width=width, taps=taps)
+    with tempfile.TemporaryDirectory() as d:
+        save_checkpoint(d, cfg, W)
+        model = registry.build_model(registry.config_from_dir(d), dtype)
+        registry.load_weights(model, d)
+    return model.to(device)
+
+
+# ---------------------------------------------------------------------------
+# boundary: gated addition, layer norm, input convolution
+# ---------------------------------------------------------------------------
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("taps", [1, 2, 4, 7])
+@pytest.mark.parametrize("sizes", [[40], [1] * 40, [2] * 20,
+                                   [3, 1, 1, 17, 2, 16]])
+def test_boundary_in_portions(device, dtype, taps, sizes):
+    """Two sequences in one batch, cut differently, the slots holding other
+    sequences' tails at first: the stream gets m * sigmoid(z + b) * d, both
+    outputs are those of whole sequences."""
+    W_, T, m = 20, 40, 0.7
+    dt = TD[dtype]
+    w, b = rnd((W_,), 1) + 1.0, rnd((W_,), 2)
+    zb, cw = rnd((W_,), 3), rnd((W_, taps), 4, 0.5)
+    state = rnd((3, taps - 1, W_), 5).to(device)
+    xs = [rnd((T, W_), 10 + i) for i in range(2)]
+    ds = [rnd((T, W_), 20 + i).to(dt) for i in range(2)]
+    zs = [rnd((T, W_), 30 + i).to(dt) for i in range(2)]
+    got_h, got_y, got_x = ([], []), ([], []), ([], [])
+    at = [0, 0]
+    plan = [(0, s) for s in sizes]
+    other = [T - 7, 1, 1, 5]
+    for i, (_, n) in enumerate(plan):
+        part = [(0, n)]
+        if i < len(other):
+            part.append((1, other[i]))
+        x = torch.cat([xs[s][at[s]:at[s] + k] for s, k in part]).to(device)
+        d = torch.cat([ds[s][at[s]:at[s] + k] for s, k in part]).to(device)
+        z = torch.cat([zs[s][at[s]:at[s] + k] for s, k in part]).to(device)
+        rows = seq_rows([(k, at[s], 2 - s) for s, k in part], device)
+        h, y = ops.add_layer_norm_conv32(
+            x, [d], [m], w.to(device), b.to(device), 1e-5, cw.to(device),
+            state, rows, dt, (z, zb.to(device)), True)
+        r0 = 0
+        for s, k in part:
+            got_h[s].append(h[r0:r0 + k].cpu())
+            got_y[s].append(y[r0:r0 + k].cpu())
+            got_x[s].append(x[r0:r0 + k].cpu())
+            at[s] += k
+            r0 += k
+    for s in range(2):
+        n = at[s]
+        x = (xs[s][:n].to(F64) + m * ds[s][:n].to(F64)
+             * torch.sigmoid(zs[s][:n].to(F64) + zb.to(F64)))
+        y = O.layer_norm(x, w, b, 1e-5)
+        assert relerr(torch.cat(got_x[s]), x) < 1e-6
+        tol = 1e-5 if dtype == "float32" else 4e-3
+        assert relerr(torch.cat(got_y[s]), y) < tol
+        assert relerr(torch.cat(got_h[s]), O.input_conv(y, cw)) < tol
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_position_rows_join_the_embedding(device, dtype):
+    emb, pos = rnd((30, 24), 1).to(TD[dtype]), rnd((50, 24), 2).to(TD[dtype])
+    tok = torch.tensor([3, 29, 0, 3, 7])
+    at = torch.tensor([0, 49, 17, 1, 2], dtype=torch.int32)
+    got = ops.embed_scale(tok.to(device), emb.to(device), 1.0,
+                          pos.to(device), at.to(device))
+    assert got.dtype == torch.float32
+    want = emb[tok].to(F64) + pos[at.long()].to(F64)
+    assert relerr(got, want) < 1e-7
+    assert relerr(ops.embed_scale(tok.to(device), emb.to(device), 2.0),
+                  2.0 * emb[tok].to(F64)) < 1e-7
+
+
+# ---------------------------------------------------------------------------
+# latent attention
+# ---------------------------------------------------------------------------
+class Harness:
+    """A mixer with a paged cache full of stale rows and scattered pages."""
+
+    def __init__(self, mx, device, dtype, n_seqs=3, max_len=320, bs=16):
+        self.mixer, self.device, self.bs = mx, device, bs
+        per = (max_len + bs - 1) // bs
+        g = torch.Generator().manual_seed(99)
+        nb = per * n_seqs + 5
+        self.tables = torch.randperm(nb, generator=g)[:per * n_seqs].view(
+            n_seqs, per).to(torch.int32)
+        kind, heads, d = mx.cache_shape()
+        assert kind == "paged"
+        self.cache = torch.randn(nb, heads, bs, d, generator=g).to(
+            dtype).to(device)
+
+    def run(self, parts):
+        """parts: [(sequence, first position, inputs [n, width])], longer
+        portions before single tokens; returns one output per part."""
+        bs, dev = self.bs, self.device
+        h = torch.cat([p for _, _, p in parts]).to(dev)
+        pos, tseq, slots, rows, r0 = [], [], [], [], 0
+        for i, (s, p0, p) in enumerate(parts):
+            for pp in range(p0, p0 + p.shape[0]):
+                pos.append(pp)
+                tseq.append(i)
+                slots.append(int(self.tables[s][pp // bs]) * bs + pp % bs)
+            rows.append([r0, p.shape[0], p0, s])
+            r0 += p.shape[0]
+        rows = torch.tensor(rows, dtype=torch.int32)
+        meta = BatchMeta(
+            positions=torch.tensor(pos, dtype=torch.int32, device=dev),
+            slot_mapping=torch.tensor(slots, dtype=torch.long, device=dev),
+            num_prefill_tokens=sum(
+                p.shape[0] for _, _, p in parts if p.shape[0] > 1),
+            prefill_token_seq=None, prefill_token_pos=None,
+            prefill_block_tables=None, num_decode_seqs=0,
+            decode_seq_lens=None, decode_block_tables=None,
+            block_tables=torch.stack(
+                [self.tables[s] for s, _, _ in parts]).to(dev),
+            token_seq=torch.tensor(tseq, dtype=torch.int32, device=dev),
+            seq_rows=rows.to(dev), seq_rows_host=rows.tolist())
+        out = self.mixer(h, meta, self.cache, {})
+        return list(out.split([p.shape[0] for _, _, p in parts]))
+
+
+SHAPES = [
+    # heads, dim, rot_dim, vdim, kv_rank, q_rank, window, scale, base
+    (3, 12, 8, 20, 24, 32, 20, 0.25, 1000.0),
+    (4, 16, 16, 8, 40, 24, 7, 0.3, 50.0),
+    (1, 8, 4, 8, 16, 8, 1, 0.5, 10.0),
+    (5, 6, 10, 7, 18, 14, 0, 0.3, 1e4),
+    (2, 24, 8, 40, 136, 16, 33, 0.2, 5e5),
+    (8, 32, 16, 32, 64, 48, 500, 0.15, 5e5),
+]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", SHAPES)
+@pytest.mark.parametrize("sizes", [[70], [1] * 70, [2] * 35,
+                                   [31, 2, 1, 1, 16, 19], [64, 6]])
+def test_latent_attention_in_portions(device, dtype, shape, sizes):
+    layer, width = mixer(*shape), 48
+    W = make_weights(make_cfg([(layer, None)], width=width), seed=31)
+    h = rnd((70, width), 32, 1.0, torch.bfloat16)
+    want = O.latent_attention(W, "l0.mix.", layer["mixer"], h.to(F64), 1e-5)
+    mx = load_layer(layer, None, W, width, dtype, device).layers[0].mixer
+    hs = Harness(mx, device, TD[dtype])
+    outs, at = [], 0
+    for n in sizes:
+        outs += hs.run([(1, at, h[at:at + n].to(TD[dtype]))])
+        at += n
+    got = torch.nn.functional.linear(torch.cat(outs), mx.out_weight)
+    assert rel_err(got, want) < TOL[dtype]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_latent_attention_ragged_batch(device, dtype):
+    """Three sequences of unequal length in shared steps, portions beside
+    single tokens, against each alone; far positions (a small rotary base
+    turns the pairs many times)."""
+    layer, width = mixer(4, 16, 8, 24, 32, 24, 40, 0.25, 20.0), 48
+    W = make_weights(make_cfg([(layer, None)], width=width), seed=16)
+    mx = load_layer(layer, None, W, width, dtype, device).layers[0].mixer
+    hs = Harness(mx, device, TD[dtype])
+    hh = [rnd((n, width), 20 + i, 1.0, torch.bfloat16)
+          for i, n in enumerate((300, 9, 151))]
+    steps = [[(0, 200), (2, 80)], [(0, 60), (2, 70), (1, 1)],
+             [(1, 2), (0, 1), (2, 1)], [(0, 39), (1, 5)], [(1, 1)]]
+    at, outs = [0, 0, 0], [[], [], []]
+    for step in steps:
+        res = hs.run([(s, at[s], hh[s][at[s]:at[s] + n].to(TD[dtype]))
+                      for s, n in step])
+        for (s, n), o in zip(step, res):
+            outs[s].append(o)
+            at[s] += n
+    assert at == [300, 9, 151]
+    for s in range(3):
+        want = O.latent_attention(W, "l0.mix.", layer["mixer"],
+                                  hh[s].to(F64), 1e-5)
+        got = torch.nn.functional.linear(torch.cat(outs[s]), mx.out_weight)
+        assert rel_err(got, want) < TOL[dtype], s
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", [(1, 1, 8), (7, 3, 20), (300, 8, 16)])
+def test_merge_heads(device, dtype, shape):
+    T, H, DV = shape
+    o = rnd((H, T, DV), 1).to(TD[dtype])
+    proj = rnd((T, H + 5), 2).to(TD[dtype])
+    g = proj[:, 5:]
+    want = (o.to(F64).transpose(0, 1)
+            * torch.sigmoid(g.to(F64)).unsqueeze(-1)).reshape(T, H * DV)
+    tol = 1e-6 if dtype == "float32" else 4e-3
+    got = ops.merge_heads(o.to(device), proj.to(device)[:, 5:])
+    assert relerr(got, want) < tol
+    flat = o.transpose(0, 1).reshape(T, H * DV).to(device)
+    ops.gate_heads(flat, proj.to(device)[:, 5:])
+    assert relerr(flat, want) < tol
+    plain = ops.merge_heads(o.to(device))
+    assert torch.equal(plain.cpu(), o.transpose(0, 1).reshape(T, H * DV))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("D", [9, 24, 72])
+def test_latent_gather(device, dtype, D):
+    cache = rnd((20, 1, 16, D), 1).to(TD[dtype])
+    tables = torch.randperm(20, generator=torch.Generator().manual_seed(2)
+                            )[:18].view(3, 6).int()
+    seg = torch.tensor([[0, 96, 0], [96, 1, 95], [97, 40, 17]],
+                       dtype=torch.int32)
+    got = ops.latent_gather(cache.to(device), tables.to(device),
+                            seg.to(device), 137, 96).cpu()
+    for i, (r0, n, p0) in enumerate(seg.tolist()):
+        for j in range(n):
+            blk, off = tables[i, (p0 + j) // 16], (p0 + j) % 16
+            assert torch.equal(got[r0 + j], cache[blk, 0, off])
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_both_forms_of_latent_attention_agree(device, dtype):
+    """The same portions through the folded and the unfolded form."""
+    layer, width = mixer(4, 16, 8, 24, 32, 24, 40, 0.25, 20.0), 48
+    W = make_weights(make_cfg([(layer, None)], width=width), seed=17)
+    mx = load_layer(layer, None, W, width, dtype, device).layers[0].mixer
+    h = rnd((150, width), 3, 1.0).to(TD[dtype])
+    outs = []
+    for ratio in (0, 1 << 20):
+        mx.EXPAND_RATIO = ratio
+        hs = Harness(mx, device, TD[dtype])
+        got = hs.run([(0, 0, h[:60])])
+        got += hs.run([(0, 60, h[60:62]), (1, 0, h[:50])])[:1]
+        got += hs.run([(0, 62, h[62:])])
+        outs.append(torch.cat(got))
+    assert rel_err(*outs) < TOL[dtype]
+    if dtype == "float32":
+        assert rel_err(*outs) > 0.0      # they are two computations
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", [(5, 24), (3, 1), (40, 1536)])
+def test_rms_norm_rows(device, dtype, shape):
+    T, C = shape
+    x, w = rnd((T, C + 7), 1, 3.0).to(TD[dtype]), rnd((C,), 2) + 1.0
+    want = O.unit_rms(x[:, 7:].to(F64), 1e-3) * w.to(F64)
+    got = ops.rms_norm_rows(x.to(device)[:, 7:], w.to(device), 1e-3)
+    assert relerr(got, want) < (1e-6 if dtype == "float32" else 4e-3)
+
+
+# ---------------------------------------------------------------------------
+# feed-forwards
+# ---------------------------------------------------------------------------
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("shape", [(9, 52), (3, 1), (20, 2048), (2, 16640),
+                                   (5, 14336)])
+def test_poly_norm(device, dtype, shape):
+    """Also rows too wide for the registers; every coefficient shows."""
+    T, F = shape
+    z = rnd((T, F + 8), 3, 1.5).to(TD[dtype])
+    tol = 2e-6 if dtype == "float32" else 4e-3
+    for coef in ([0.7, -0.4, 0.5, 0.2], [1, 0, 0, 0], [0, 1, 0, 0],
+                 [0, 0, 1, 0], [0, 0, 0, 1]):
+        c = torch.tensor(coef, dtype=torch.float32)
+        want = O.poly_norm(z[:, 8:].to(F64), c, 1e-5)
+        got = ops.poly_norm(z.to(device)[:, 8:], c.to(device), 1e-5)
+        assert relerr(got, want) < tol, coef
+
+
+def run_ff(model, x, ids, small):
+    layer = model.layers[0]
+    plan = None
+    if layer.spec.mlp.kind == "moe":
+        plan = TablePlans([layer.mlp]).plan(ids, not small)[0]
+    return layer.feed_forward(x, small, plan)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_dense_feed_forward_and_gate(device, dtype):
+    W = make_weights(make_cfg([(mixer(), dense(56))]), seed=3)
+    model = load_layer(mixer(), dense(56), W, 64, dtype, device)
+    h = rnd((23, 64), 5, 1.0, torch.bfloat16)
+    y, z = run_ff(model, h.to(TD[dtype]).to(device), None, True)
+    assert rel_err(y.float(), O.dense_ff(W, "l0.mlp.", h.to(F64), 1e-5)) \
+        < TOL[dtype]
+    got = torch.sigmoid(z.float() + model.layers[0].rg2_b)
+    assert relerr(got, O.gate(W, "l0.rg2", h.to(F64))) < (
+        1e-5 if dtype == "float32" else 1e-2)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("small", [True, False])
+@pytest.mark.parametrize("shape", [(24, 5, 2), (8, 1, 1), (20, 3, 3),
+                                   (16, 40, 1), (40, 6, 4)])
+def test_table_routed_experts(device, dtype, small, shape):
+    """Both dispatch forms (grouped kernels / one GEMM pair per expert), few
+    and many rows per expert, experts nobody chose, widths that are and are
+    not whole vectors."""
+    mlp = moe(*shape)
+    W = make_weights(make_cfg([(mixer(), mlp)]), seed=8)
+    model = load_layer(mixer(), mlp, W, 64, dtype, device)
+    for n in (1, 7, 150):
+        h = rnd((n, 64), 40 + n, 1.0, torch.bfloat16)
+        ids = torch.randint(0, 97, (n,),
+                            generator=torch.Generator().manual_seed(n))
+        want = O.table_ff(W, "l0.mlp.", mlp, h.to(F64), ids)
+        y, _ = run_ff(model, h.to(TD[dtype]).to(device), ids.to(device),
+                      small)
+        assert y.dtype == torch.float32
+        assert rel_err(y, want) < TOL[dtype], n
+
+
+def check_plan(sel, n_out, offs, rows, pos):
+    T, top = sel.shape
+    flat = sel.flatten().tolist()
+    order = sorted(range(T * top), key=lambda i: flat[i])   # stable
+    assert rows.tolist() == [i // top for i in order]
+    back = [0] * (T * top)
+    for p, i in enumerate(order):
+        back[i] = p
+    assert pos.tolist() == back
+    want = [0]
+    for e in range(n_out):
+        want.append(want[-1] + flat.count(e))
+    assert offs.tolist() == want
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("shape", [(1, 1, 1), (5, 2, 3), (64, 2, 8),
+                                   (200, 3, 300), (1500, 4, 17),
+                                   (9, 1, 1000)])
+def test_expert_plan_is_a_stable_sort(device, shape):
+    T, top, n_out = shape
+    g = torch.Generator().manual_seed(T)
+    sel = torch.randint(0, n_out, (T, top), generator=g)
+    # skewed: one output takes many entries
+    sel[torch.rand(T, top, generator=g) < 0.3] = n_out // 2
+    got = [t.cpu() for t in ops.expert_plan(sel.to(device), n_out)]
+    check_plan(sel, n_out, *got)
+    # the table form: three layers at once
+    tables = torch.randint(0, n_out, (3, 29, top), generator=g).to(
+        torch.int32)
+    tok = torch.randint(0, 29, (T,), generator=g)
+    offs, rows, pos = ops.table_plan(tok.to(device), tables.to(device),
+                                     n_out)
+    for j in range(3):
+        check_plan(tables[j][tok].long(), n_out, offs[j].cpu(),
+                   rows[j].cpu(), pos[j].cpu())
+
+
+# ---------------------------------------------------------------------------
+# kernels against the reference ops
+# ---------------------------------------------------------------------------
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W_", [64, 60, 2048, 8200])
+@pytest.mark.parametrize("taps", [0, 1, 3, 4, 9])
+@pytest.mark.parametrize("kind", ["single", "ragged"])
+def test_gated_boundary_kernel(dtype, W_, taps, kind):
+    """One-launch form of single-row segments and the two-launch form of
+    ragged batches; deltas of the serving dtype and fp32; row-strided gate
+    and delta views; rows wider than the registers hold."""
+    dt = TD[dtype]
+    parts = ([(1, 5, 2), (1, 0, 0), (1, 1, 3), (1, 70, 1)]
+             if kind == "single" else
+             [(70, 0, 2), (2, 9, 0), (1, 4, 3), (130, 3, 1)])
+    T = sum(p[0] for p in parts)
+    x = rnd((T, W_), 1)
+    w, b, zb = rnd((W_,), 2) + 1.0, rnd((W_,), 3), rnd((W_,), 4)
+    cw = rnd((W_, taps), 5, 0.5) if taps else None
+    st = rnd((5, max(taps - 1, 0), W_), 6)
+    z = rnd((T, W_ + 8), 7).to(dt)
+    rows = seq_rows(parts)
+    for ddt in {dt, torch.float32}:
+        d = rnd((T, W_ + 8), 8).to(ddt)
+        for plain in (False, True):
+            xr, sr = x.clone(), st.clone()
+            want = R.add_layer_norm_conv32(
+                xr, [d[:, 8:]], [0.7], w, b, 1e-5, cw, sr, rows, dt,
+                (z[:, 8:], zb), plain)
+            xg, sg = x.cuda(), st.cuda()
+            got = ops.add_layer_norm_conv32(
+                xg, [d.cuda()[:, 8:]], [0.7], w.cuda(), b.cuda(), 1e-5,
+                cw.cuda() if taps else None, sg if taps else None,
+                rows.cuda(), dt, (z.cuda()[:, 8:], zb.cuda()), plain)
+            tol = 1e-5 if dtype == "float32" else 4e-3
+            for a, e in zip(*(([got], [want]) if not plain
+                              else (got, want))):
+                assert relerr(a, e) < tol
+            assert relerr(xg, xr) < 1e-6
+            if taps > 1:
+                assert relerr(sg, sr) < 1e-5
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("act,gated", [("silu", True), ("gelu_tanh", True),
+                                       ("clamped_swish", True),
+                                       ("relu2", False), ("silu", False)])
+@pytest.mark.parametrize("shape", [
+    # rows, width, ff, experts, top
+    (1, 64, 24, 3, 1), (13, 200, 72, 5, 2), (64, 520, 136, 8, 2),
+    (128, 256, 64, 3, 3), (300, 64, 96, 2, 2), (40, 1096, 8, 30, 4)])
+def test_grouped_experts_kernel(act, gated, shape):
+    """Segments of 0 to several hundred rows, reduction lengths below,
+    at and above a chunk of 256 with remainders, output widths that fill no
+    tile; with and without a scale on the inputs."""
+    T, W_, ff, E, top = shape
+    g = torch.Generator().manual_seed(T + W_)
+    bf = torch.bfloat16
+    x = rnd((T, W_), 1, 1.0, bf)
+    w_in = rnd((E, (2 if gated else 1) * ff, W_), 2, W_ ** -0.5, bf)
+    w_out = rnd((E, W_, ff), 3, ff ** -0.5, bf)
+    sel = torch.rand(T, E, generator=g).topk(top, dim=1).indices
+    if E > 2:
+        sel[sel == 1] = 0                      # nobody chooses expert 1
+    offs, rows, pos = ops.expert_plan(sel, E)
+    for scale in (None, torch.rand(T * top, generator=g) + 0.5):
+        want = ops.experts_grouped(x, w_in, w_out, offs, rows, act, 1.5,
+                                   gated, scale)
+        got = ops.experts_grouped(
+            x.cuda(), w_in.cuda(), w_out.cuda(), offs.cuda(), rows.cuda(),
+            act, 1.5, gated, scale.cuda() if scale is not None else None)
+        assert rel_err(got.float(), want.float()) < 2e-2
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W_", [64, 61])
+def test_experts_sum_kernel(dtype, W_):
+    T, top, E = 37, 3, 4
+    dt = TD[dtype]
+    g = torch.Generator().manual_seed(5)
+    sel = torch.rand(T, E + 2, generator=g).topk(top, dim=1).indices
+    _, _, pos = ops.expert_plan(sel, E + 2)
+    ys, x = rnd((T * top, W_), 1).to(dt), rnd((T, W_), 2).to(dt)
+    wts = torch.rand(T, top, generator=g)
+    sy, sg = rnd((T, W_), 3).to(dt), rnd((T, 1), 4).to(dt)
+
+    def c(t):
+        return t.cuda() if t is not None else None
+
+    for weights, s, a, b in ((wts, sel, sy, sg), (None, None, None, None),
+                             (wts, None, sy, None)):
+        want = R.experts_sum(ys, pos, top, weights, 0.25, s, E, x, a, b)
+        got = ops.experts_sum(c(ys), c(pos), top, c(weights), 0.25, c(s), E,
+                              c(x), c(a), c(b))
+        assert got.dtype == torch.float32 and relerr(got, want) < 1e-6
