@@ -399,8 +399,8 @@ __global__ __launch_bounds__(256) void mfma_attn_combine_kernel(
 }
 
 static size_t mf_lds_budget(const void* fn) {
-  // 160 KB per CU less the kernel's static arrays
-  const int want = 160 * 1024 - 1024;
+  // 160 KB per CU less the kernel's static arrays (1.5 KB with 128 rows)
+  const int want = 160 * 1024 - 2048;
   if (hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize,
                           want) == hipSuccess)
     return (size_t)want;

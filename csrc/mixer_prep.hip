@@ -307,15 +307,22 @@ __global__ __launch_bounds__(256) void merge_heads_kernel(
 }
 
 // One wave per row: segment blockIdx.y's row r comes from position p0 + r of
-// its sequence. U: copy unit.
+// its sequence; the rows up to the next multiple of `pad` are zero-filled.
+// U: copy unit.
 template <typename U>
 __global__ __launch_bounds__(256) void latent_gather_kernel(
     U* __restrict__ out, const U* __restrict__ cache,
     const int* __restrict__ block_tables, int max_blocks,
-    const int* __restrict__ segments, int BS, int units) {
+    const int* __restrict__ segments, int BS, int units, int pad) {
   const int* sg = segments + 3 * blockIdx.y;
   const int r = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (r >= sg[1]) return;
+  if (r >= sg[1]) {
+    if (r < (sg[1] + pad - 1) / pad * pad) {
+      U* dst = out + ((int64_t)sg[0] + r) * units;
+      for (int c = threadIdx.x & 63; c < units; c += 64) dst[c] = U();
+    }
+    return;
+  }
   const int p = sg[2] + r;
   const int blk = block_tables[(size_t)blockIdx.y * max_blocks + p / BS];
   const U* src = cache + ((int64_t)blk * BS + p % BS) * units;
@@ -483,15 +490,16 @@ void mx_merge_heads(void* out, int ldo, const void* o, int hs, int rs,
 
 void mx_latent_gather(void* out, const void* cache, const void* block_tables,
                       int max_blocks, const void* segments, int S_,
-                      int longest, int BS, int D, int dtype, void* stream) {
-  if (S_ <= 0 || longest <= 0) return;
+                      int longest, int BS, int D, int pad, int dtype,
+                      void* stream) {
+  if (S_ <= 0 || longest <= 0 || pad < 1) return;
   const int bytes = D * (dtype == MX_BF16 ? 2 : 4);
-  dim3 grid((longest + 3) / 4, S_);
+  dim3 grid(((longest + pad - 1) / pad * pad + 3) / 4, S_);
 #define LG_GO(U)                                                            \
   hipLaunchKernelGGL((latent_gather_kernel<U>), grid, dim3(256), 0,         \
                      (hipStream_t)stream, (U*)out, (const U*)cache,         \
                      (const int*)block_tables, max_blocks,                  \
-                     (const int*)segments, BS, bytes / (int)sizeof(U))
+                     (const int*)segments, BS, bytes / (int)sizeof(U), pad)
   if (bytes % 16 == 0 && (((size_t)out | (size_t)cache) & 15) == 0)
     LG_GO(uint4);
   else

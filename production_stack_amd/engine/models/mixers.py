@@ -19,10 +19,12 @@ Each mixer exposes
 from __future__ import annotations
 
 import math
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
 import torch.nn as nn
+import torch.nn.functional as F
 
 from production_stack_amd import ops
 from production_stack_amd.engine.config import MixerSpec
@@ -202,6 +204,64 @@ class TalkAttention(nn.Module):
         return out
 
 
+@dataclass
+class _Expansion:
+    """A step's prompt portions for unfolded latent attention. Segment i
+    (the i-th portion) sees `rows` cached rows from position `lo` on; they
+    are laid down from a multiple of EXPAND_PAD on."""
+
+    segments: torch.Tensor       # int32 [S, 3]: first row, rows, lo
+    tiles: torch.Tensor          # int32 [NT, 4], see ops.expanded_attention
+    total: int                   # rows, padding included
+    longest: int                 # rows of the longest segment
+    tokens: int                  # query rows
+    pages: Optional[tuple] = None
+
+    @classmethod
+    def build(cls, host, npt: int, window: int, meta,
+              ratio: int) -> Optional["_Expansion"]:
+        """host: the step's (first row, rows, first position, slot) rows,
+        portions first; None where the visible keys outnumber `ratio` times
+        the portions' tokens."""
+        pad, step = ops.EXPAND_PAD, ops.EXPAND_TILE
+        segs, tiles, at, rows, keys = [], [], 0, 0, 0
+        for _, n, p0, _ in host:
+            if rows >= npt:
+                break
+            lo = max(0, p0 - window + 1) if window else 0
+            seen = p0 + n - lo
+            segs.append((at, seen, lo))
+            tiles += [(rows + t, min(step, n - t), at, p0 - lo + t)
+                      for t in range(0, n, step)]
+            at += -(-seen // pad) * pad
+            rows += n
+            keys += seen
+        if rows != npt or keys > ratio * npt:
+            return None
+        # tiles that see the most keys go first
+        tiles.sort(key=lambda t: -(min(t[3], window) if window else t[3]))
+        dev = meta.positions.device
+        return cls(
+            torch.tensor(segs, dtype=torch.int32).to(dev, non_blocking=True),
+            torch.tensor(tiles, dtype=torch.int32).to(dev,
+                                                      non_blocking=True),
+            at, max(s[1] for s in segs), npt)
+
+    def rows_as_pages(self, meta):
+        """The expanded rows as a cache of one-row pages: (block table int32
+        [S, longest], query positions counted from the segments' first
+        rows)."""
+        if self.pages is None:
+            seg = self.segments
+            table = (seg[:, :1] + torch.arange(
+                self.longest, dtype=torch.int32,
+                device=seg.device)).clamp_(max=self.total - 1)
+            n = self.tokens
+            pos = meta.positions[:n] - seg[:, 2][meta.token_seq[:n].long()]
+            self.pages = (table, pos)
+        return self.pages
+
+
 class LatentAttention(nn.Module):
     """Multi-head attention whose keys and values are low-rank expansions
     of one cached latent per token. Per head the query has `dim`
@@ -298,45 +358,50 @@ class LatentAttention(nn.Module):
             w = self._unfolded = (k.view(H * (D + R), L + R), v)
         return w
 
-    def _expansion(self, meta, npt: int, shared: dict):
-        """The step's plan of expanded prompt portions (None: folded form):
-        (segment table int32 [S, 3] = first expanded row, rows, first
-        position; rows in all, longest segment, row table [S, longest],
-        positions counted from the segments' first rows). Layers with one
-        window share it."""
+    def _expansion(self, meta, npt: int,
+                   shared: dict) -> Optional[_Expansion]:
+        """The step's plan of expanded prompt portions (None: folded form);
+        layers with one window share it."""
         host = getattr(meta, "seq_rows_host", None)
         if host is None or npt == 0:
             return None
         win = self.spec.window
         key = ("latent_expansion", win)
         if key not in shared:
-            segs, at, rows = [], 0, 0
-            for _, n, p0, _ in host:
-                if rows >= npt:
-                    break
-                lo = max(0, p0 - win + 1) if win else 0
-                segs.append((at, p0 + n - lo, lo))
-                at += p0 + n - lo
-                rows += n
-            plan = None
-            if rows == npt and at <= self.EXPAND_RATIO * npt:
-                dev = meta.positions.device
-                seg = torch.tensor(segs, dtype=torch.int32).to(
-                    dev, non_blocking=True)
-                longest = max(s[1] for s in segs)
-                table = (seg[:, :1] + torch.arange(
-                    longest, dtype=torch.int32, device=dev)).clamp_(
-                        max=at - 1)
-                pos = meta.positions[:npt] - seg[:, 2][
-                    meta.token_seq[:npt].long()]
-                plan = (seg, at, longest, table, pos)
-            shared[key] = plan
+            shared[key] = _Expansion.build(host, npt, win, meta,
+                                           self.EXPAND_RATIO)
         plan = shared[key]
         if plan is not None:
-            size = plan[1] * self.H * (self.D + self.R + self.DV)
+            size = plan.total * self.H * (self.D + self.R + self.DV)
             if size * self.uk.element_size() > self.EXPAND_BYTES:
                 return None
         return plan
+
+    def _attend_expanded(self, q, plan, meta, cache, gate, out) -> None:
+        """Attention of the portions' queries q [n, H*(dim+rot_dim)] over
+        expanded keys and values, head gates included."""
+        H, D, R, L, DV = self.H, self.D, self.R, self.L, self.DV
+        sp, n, N = self.spec, q.shape[0], plan.total
+        rows = ops.latent_gather(cache, meta.block_tables, plan.segments, N,
+                                 plan.longest)
+        wk, wv = self.unfolded()
+        k = F.linear(rows, wk)
+        if ops.expanded_attention_fits(q, D + R, DV, sp.softcap):
+            # the values come out transposed, as that kernel reads them
+            vt = F.linear(wv, rows[:, :L])
+            ops.expanded_attention(
+                q, k, vt, plan.tiles, self.scale, H, window=sp.window,
+                sink=sp.sink, sink_vals=self.sink_vals, gate=gate, out=out)
+            return
+        v = F.linear(rows[:, :L], wv)
+        table, pos = plan.rows_as_pages(meta)
+        ops.talk_attention(
+            q, k.view(N, H, 1, D + R), v.view(N, H, 1, DV), table,
+            meta.token_seq[:n], pos, self.scale, H, window=sp.window,
+            sink=sp.sink, out=out, softcap=sp.softcap,
+            sink_vals=self.sink_vals)
+        if gate is not None:
+            ops.gate_heads(out, gate)
 
     @property
     def out_in(self) -> int:
@@ -377,19 +442,9 @@ class LatentAttention(nn.Module):
             ops.latent_prep(None, qn, dkv[:n], self.latent_norm, self.eps,
                             cs, meta.positions[:n], cache,
                             meta.slot_mapping[:n], H, D, R, rd)
-            seg, total, longest, table, pos = plan
-            rows = ops.latent_gather(cache, meta.block_tables, seg, total,
-                                     longest)
-            wk, wv = self.unfolded()
-            k = gemm_policy.linear(rows, wk)
-            v = gemm_policy.linear(rows[:, :L], wv)
-            ops.talk_attention(
-                qn, k.view(total, H, 1, D + R), v.view(total, H, 1, DV),
-                table, meta.token_seq[:n], pos, self.scale, H,
-                window=sp.window, sink=sp.sink, out=o[:n],
-                softcap=sp.softcap, sink_vals=self.sink_vals)
-            if gate is not None:
-                ops.gate_heads(o[:n], gate[:n])
+            self._attend_expanded(qn, plan, meta, cache,
+                                  gate[:n] if gate is not None else None,
+                                  o[:n])
         if n == T:
             return o
         # position-free query part into the latent space: [H, T, L]

@@ -966,18 +966,27 @@ def gate_heads(o: torch.Tensor, gate: torch.Tensor) -> None:
                          _stream())
 
 
+# expanded rows of a segment start at multiples of this many rows
+EXPAND_PAD = 64
+# query rows of an expanded-attention tile
+EXPAND_TILE = 128
+
+
 def latent_gather(cache: torch.Tensor, block_tables: torch.Tensor,
                   segments: torch.Tensor, total: int,
                   longest: int) -> torch.Tensor:
     """Rows of a paged cache [NB, 1, BS, D] side by side: segments int32
     [S, 3] = (first output row, rows, first position) of the sequences whose
-    block tables are block_tables[:S]; together they fill `total` rows, the
-    longest has `longest`. Returns [total, D]."""
+    block tables are block_tables[:S]. First output rows are multiples of
+    EXPAND_PAD, every segment is zero-filled up to the next one; together
+    they fill `total` rows, the longest has `longest`. Returns
+    [total, D]."""
     NB, one, BS, D = cache.shape
     S = segments.shape[0]
     assert one == 1 and block_tables.dtype == torch.int32
     assert block_tables.dim() == 2 and block_tables.shape[0] >= S
     assert segments.dtype == torch.int32 and segments.shape[1] == 3
+    assert total % EXPAND_PAD == 0
     if not cache.is_cuda:
         return reference.latent_gather(cache, block_tables, segments, total)
     assert cache.is_contiguous() and block_tables.is_contiguous()
@@ -985,7 +994,64 @@ def latent_gather(cache: torch.Tensor, block_tables: torch.Tensor,
     out = torch.empty((total, D), dtype=cache.dtype, device=cache.device)
     _mx().mx_latent_gather(
         _p(out), _p(cache), _p(block_tables), block_tables.shape[1],
-        _p(segments), S, longest, BS, D, _mx_dtype(cache.dtype), _stream())
+        _p(segments), S, longest, BS, D, EXPAND_PAD, _mx_dtype(cache.dtype),
+        _stream())
+    return out
+
+
+def expanded_attention_fits(q: torch.Tensor, dim: int, vdim: int,
+                            softcap: float = 0.0) -> bool:
+    """Whether expanded_attention covers these queries and head widths."""
+    return (q.dtype == torch.bfloat16 and dim % 8 == 0 and dim <= 192
+            and vdim <= 128 and softcap == 0.0 and q.stride(0) % 8 == 0
+            and q.data_ptr() % 16 == 0)
+
+
+def expanded_attention(q: torch.Tensor, k: torch.Tensor, vt: torch.Tensor,
+                       tiles: torch.Tensor, scale: float, heads: int,
+                       window: int = 0, sink: bool = False,
+                       sink_vals: torch.Tensor = None,
+                       gate: torch.Tensor = None,
+                       out: torch.Tensor = None) -> torch.Tensor:
+    """Causal attention of prompt portions, every head with keys and values
+    of its own. q [T, H*D] row-strided; k [N, H*D]; vt [H*DV, N] (values
+    transposed); tiles int32 [NT, 4] = (first query row, rows up to
+    EXPAND_TILE, first key row of the segment, the first query's position
+    counted from there): query row r of a tile sees the key rows j <= its
+    position p of its segment with p - j < window (0: all); sink as in
+    talk_attention; gate [T, H] row-strided: head outputs times
+    sigmoid(gate). bfloat16; see expanded_attention_fits. A segment's key
+    rows are zero-filled up to a multiple of EXPAND_PAD."""
+    T = q.shape[0]
+    H = heads
+    N = k.shape[0]
+    D, DV = k.shape[1] // H, vt.shape[0] // H
+    assert q.shape == (T, H * D) and k.shape == (N, H * D)
+    assert vt.shape == (H * DV, N) and N % EXPAND_PAD == 0
+    assert tiles.dtype == torch.int32 and tiles.shape[1] == 4
+    assert k.dtype == q.dtype and vt.dtype == q.dtype
+    if sink_vals is not None:
+        assert sink and sink_vals.dtype == torch.float32
+        assert sink_vals.shape == (H,)
+    if gate is not None:
+        assert gate.shape == (T, H) and gate.dtype == q.dtype
+    if out is None:
+        out = torch.empty((T, H * DV), dtype=q.dtype, device=q.device)
+    assert out.shape == (T, H * DV) and out.dtype == q.dtype
+    if not q.is_cuda:
+        out.copy_(reference.expanded_attention(
+            q, k, vt, tiles, scale, H, window, sink, sink_vals, gate))
+        return out
+    assert k.is_contiguous() and vt.is_contiguous()
+    assert tiles.is_contiguous()
+    rc = _mx().mx_expand_attention(
+        _p(out), _rows(out, "out"), _p(q), _rows(q, "q"), _p(k), _p(vt), N,
+        _p(tiles), tiles.shape[0], H, D, DV, _f(scale), int(window),
+        int(bool(sink)), _p(sink_vals), _p(gate),
+        _rows(gate, "gate") if gate is not None else 0, _stream())
+    if rc != 0:
+        raise RuntimeError(
+            f"expanded_attention: head widths {D}/{DV} are not built")
     return out
 
 

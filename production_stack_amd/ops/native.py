@@ -10,7 +10,8 @@ shape checks live in the Python wrappers
 
 Groups (one shared library each):
   core    resid32, norm_conv, mixer_prep, talk_attention, mfma_attention,
-          moe_route, moe_group, mingru_scan -> _mixops.so
+          expand_attention, moe_route, moe_group, mingru_scan
+                                            -> _mixops.so
   delta   delta_rule                        -> _mixops_delta.so
   gdelta  gated_delta                       -> _mixops_gdelta.so
   scan    linear_scan                       -> _mixops_scan.so
@@ -45,6 +46,7 @@ GROUPS = {
         ("talk_attention.hip", []),
         ("mixer_prep.hip", []),
         ("mfma_attention.hip", []),
+        ("expand_attention.hip", []),
         ("moe_route.hip", []),
         ("moe_group.hip", []),
         ("mingru_scan.hip", []),
@@ -81,7 +83,7 @@ INT_RESULT = {
     "mx_delta_rule", "mx_talk_attention", "mx_gated_delta",
     "mx_short_conv_silu", "mx_mfma_attention", "mx_linear_scan",
     "mx_linear_scan_splits", "mx_norm_conv32", "mx_moe_route",
-    "mx_add_layer_norm32", "mx_expert_plan",
+    "mx_add_layer_norm32", "mx_expert_plan", "mx_expand_attention",
 }
 
 # entry points that return a 64-bit count

@@ -618,13 +618,45 @@ def latent_prep(q_lat, q, dkv, norm_w, eps: float, cos_sin, positions,
 
 def latent_gather(cache, block_tables, segments, total: int):
     """[total, D]: cached rows of the segments (first output row, rows,
-    first position), segment i through block_tables[i]."""
+    first position), segment i through block_tables[i], zeros between
+    them."""
     bs = cache.shape[2]
-    out = torch.empty((total, cache.shape[3]), dtype=cache.dtype)
+    out = torch.zeros((total, cache.shape[3]), dtype=cache.dtype)
     for i, (r0, n, p0) in enumerate(segments.tolist()):
         p = torch.arange(p0, p0 + n)
         out[r0:r0 + n] = cache[block_tables[i, p // bs].long(), 0, p % bs]
     return out
+
+
+def expanded_attention(q, k, vt, tiles, scale: float, heads: int,
+                       window: int, sink: bool, sink_vals, gate):
+    """Causal windowed attention of tiles of consecutive query rows over
+    their segment's key rows k [N, H*D] and transposed values vt [H*DV, N];
+    fp32 scores and weights. Rows outside every tile are zero."""
+    T, N, H = q.shape[0], k.shape[0], heads
+    D, DV = k.shape[1] // H, vt.shape[0] // H
+    kf = k.float().view(N, H, D)
+    vf = vt.float().view(H, DV, N)
+    out = torch.zeros(T, H, DV)
+    for r0, n, k0, p0 in tiles.tolist():
+        last = p0 + n
+        s = torch.einsum("thd,jhd->htj", q[r0:r0 + n].float().view(n, H, D),
+                         kf[k0:k0 + last]) * scale
+        age = (p0 + torch.arange(n))[:, None] - torch.arange(last)[None, :]
+        seen = age >= 0
+        if window > 0:
+            seen &= age < window
+        s = s.masked_fill(~seen, float("-inf"))
+        if sink:
+            sv = (sink_vals if sink_vals is not None
+                  else torch.zeros(H)).float()
+            s = torch.cat([s, sv.view(H, 1, 1).expand(H, n, 1)], dim=-1)
+        w = torch.softmax(s, dim=-1)[..., :last]
+        out[r0:r0 + n] = torch.einsum("htj,hdj->thd", w,
+                                      vf[:, :, k0:k0 + last])
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float()).unsqueeze(-1)
+    return out.reshape(T, H * DV).to(q.dtype)
 
 
 def short_conv_silu(x, w, state, seq_rows, out_dtype, bias=None):

@@ -258,10 +258,11 @@ def test_latent_gather(device, dtype, D):
     cache = rnd((20, 1, 16, D), 1).to(TD[dtype])
     tables = torch.randperm(20, generator=torch.Generator().manual_seed(2)
                             )[:18].view(3, 6).int()
-    seg = torch.tensor([[0, 96, 0], [96, 1, 95], [97, 40, 17]],
+    seg = torch.tensor([[0, 96, 0], [128, 1, 95], [192, 64, 17]],
                        dtype=torch.int32)
     got = ops.latent_gather(cache.to(device), tables.to(device),
-                            seg.to(device), 137, 96).cpu()
+                            seg.to(device), 256, 96).cpu()
+    assert not got[96:128].any() and not got[129:192].any()
     for i, (r0, n, p0) in enumerate(seg.tolist()):
         for j in range(n):
             blk, off = tables[i, (p0 + j) // 16], (p0 + j) % 16
@@ -445,6 +446,56 @@ def test_gated_boundary_kernel(dtype, W_, taps, kind):
             assert relerr(xg, xr) < 1e-6
             if taps > 1:
                 assert relerr(sg, sr) < 1e-5
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("shape", [
+    # heads, key width, value width, window, sink, scale
+    (3, 24, 20, 0, None, 0.3), (8, 192, 128, 70, None, 0.1),
+    (2, 64, 64, 1, None, 0.3), (5, 96, 33, 64, "learned", 0.2),
+    (16, 128, 128, 200, "zero", 0.1), (1, 136, 72, 129, None, 0.2),
+    (8, 40, 128, 1000, "learned", 0.3)])
+def test_expanded_attention_kernel(shape):
+    """Segments with and without history, tiles of 1 to 128 rows, a key
+    that stands out at every distance around the window's edge."""
+    H, D, DV, win, sink, scale = shape
+    bf = torch.bfloat16
+    segs = [(0, 300), (130, 131), (5, 2), (64, 64), (0, 127)]  # (past, rows)
+    tiles, T, N = [], 0, 0
+    for past, n in segs:
+        for t in range(0, n, 128):
+            tiles.append((T + t, min(128, n - t), N, past + t))
+        T += n
+        N += -(-(past + n) // 64) * 64
+    q, k = rnd((T, H * D + 8), 1, 1.0, bf)[:, 8:], rnd((N, H * D), 2, 1.0, bf)
+    vt = rnd((H * DV, N), 3, 1.0, bf)
+    at = 0
+    for past, n in segs:       # zero-filled padding
+        end = at + past + n
+        nxt = at + -(-(past + n) // 64) * 64
+        k[end:nxt] = 0
+        vt[:, end:nxt] = 0
+        at = nxt
+    # the query of row 250 of the first segment matches one key strongly
+    g = rnd((T, H), 4, 1.0, bf)
+    sv = rnd((H,), 5) if sink == "learned" else None
+    spots = [250 - max(win, 60) + 1, 250 - max(win, 60), 250, 128, 0]
+    for spot in [None] + [s for s in spots if s >= 0]:
+        kk = k.clone()
+        if spot is not None:
+            kk[spot] = q[250] * 2
+        for gate in (None, g):
+            want = R.expanded_attention(q, kk, vt, torch.tensor(tiles),
+                                        scale, H, win, bool(sink), sv, gate)
+            got = ops.expanded_attention(
+                q.cuda(), kk.cuda(), vt.cuda(),
+                torch.tensor(tiles, dtype=torch.int32).cuda(), scale, H,
+                window=win, sink=bool(sink),
+                sink_vals=sv.cuda() if sv is not None else None,
+                gate=gate.cuda() if gate is not None else None)
+            err = (got.cpu().float() - want.float()).norm(dim=-1) / \
+                want.float().norm(dim=-1)
+            assert float(err.max()) < 1e-2, (spot, gate is None)
 
 
 @pytest.mark.gpu
