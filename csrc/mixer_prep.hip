@@ -191,29 +191,34 @@ PS_DEV void mx_turn(float u, float w, const float* cs, float* ou, float* ow) {
   *ow = w * cs[0] + u * cs[1];
 }
 
-template <typename T>
+// Grid (tokens, 1 + head groups): workgroup y = 0 normalises the latent,
+// turns the shared key part and appends the row; workgroup y > 0 assembles
+// the queries of HG heads. VEC: latent parts are whole 16-byte vectors.
+#define LP_HG 4
+
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void latent_prep_kernel(
-    T* qf, const T* __restrict__ qlat, const T* q, int ldq, const T* __restrict__ dkv, int lddkv,
-    const float* __restrict__ normw, float eps,
-    const float* __restrict__ cos_sin, int table_rows, int rot_dims,
-    const int* __restrict__ positions, T* __restrict__ cache,
-    const int64_t* __restrict__ slots, int T_, int H, int D, int R, int L,
-    int BS) {
+    T* qf, const T* __restrict__ qlat, const T* q, int ldq,
+    const T* __restrict__ dkv, int lddkv, const float* __restrict__ normw,
+    float eps, const float* __restrict__ cos_sin, int table_rows,
+    int rot_dims, const int* __restrict__ positions, T* __restrict__ cache,
+    const int64_t* __restrict__ slots, int T_, int H, int D, int R, int L) {
   __shared__ float red[17];
   const int t = blockIdx.x;
   const int pos = min(max(positions[t], 0), table_rows - 1);
   const float* cs = cos_sin + (size_t)pos * rot_dims;  // [rot_dims/2][2]
-  const T* row = dkv + (size_t)t * lddkv;
-  const int64_t slot = slots[t];
-  T* crow = cache + (slot >= 0 ? slot : 0) * (int64_t)(L + R);
-  float ss = 0.f;
-  for (int c = threadIdx.x; c < L; c += blockDim.x) {
-    const float x = MxElem<T>::ld(row + c);
-    ss += x * x;
-  }
-  ss = mx_block_sum(ss, red);
-  const float inv = 1.0f / sqrtf(ss / (float)L + eps);
-  if (slot >= 0) {
+  if (blockIdx.y == 0) {
+    const T* row = dkv + (size_t)t * lddkv;
+    const int64_t slot = slots[t];
+    T* crow = cache + (slot >= 0 ? slot : 0) * (int64_t)(L + R);
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < L; c += blockDim.x) {
+      const float x = MxElem<T>::ld(row + c);
+      ss += x * x;
+    }
+    ss = mx_block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)L + eps);
+    if (slot < 0) return;
     for (int c = threadIdx.x; c < L; c += blockDim.x)
       MxElem<T>::st(crow + c, MxElem<T>::ld(row + c) * inv * normw[c]);
     // shared key part: pairs below rot_dims turn, the rest passes
@@ -224,15 +229,16 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
       MxElem<T>::st(crow + L + 2 * i, u);
       MxElem<T>::st(crow + L + 2 * i + 1, w);
     }
-    if ((R & 1) && threadIdx.x == 0)
-      crow[L + R - 1] = row[L + R - 1];
+    if ((R & 1) && threadIdx.x == 0) crow[L + R - 1] = row[L + R - 1];
+    return;
   }
+  const int h0 = (blockIdx.y - 1) * LP_HG, hn = min(LP_HG, H - h0);
   if (qlat == nullptr) {
     // queries stay as they are, their rotary parts turn in place (qf is q);
     // a thread owns both entries of a pair
-    for (int c = threadIdx.x; c < H * (rot_dims / 2); c += blockDim.x) {
+    for (int c = threadIdx.x; c < hn * (rot_dims / 2); c += blockDim.x) {
       const int h = c / (rot_dims / 2), i = c - h * (rot_dims / 2);
-      T* p = qf + (size_t)t * ldq + h * (D + R) + D + 2 * i;
+      T* p = qf + (size_t)t * ldq + (h0 + h) * (D + R) + D + 2 * i;
       float u, w;
       mx_turn(MxElem<T>::ld(p), MxElem<T>::ld(p + 1), cs + 2 * i, &u, &w);
       MxElem<T>::st(p, u);
@@ -242,24 +248,35 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
   }
   // queries: per head [latent-space part | turned rotary part]
   const int QW = L + R;
-  for (int c = threadIdx.x; c < H * L; c += blockDim.x) {
-    const int h = c / L, l = c - h * L;
-    qf[(size_t)t * H * QW + h * QW + l] = qlat[((size_t)h * T_ + t) * L + l];
+  T* qrow = qf + (size_t)t * H * QW + (size_t)h0 * QW;
+  if (VEC) {
+    constexpr int V = 16 / sizeof(T);
+    const int n = L / V;
+    for (int c = threadIdx.x; c < hn * n; c += blockDim.x) {
+      const int h = c / n, l = (c - h * n) * V;
+      *(uint4*)(qrow + h * QW + l) =
+          *(const uint4*)(qlat + ((size_t)(h0 + h) * T_ + t) * L + l);
+    }
+  } else {
+    for (int c = threadIdx.x; c < hn * L; c += blockDim.x) {
+      const int h = c / L, l = c - h * L;
+      qrow[h * QW + l] = qlat[((size_t)(h0 + h) * T_ + t) * L + l];
+    }
   }
-  for (int c = threadIdx.x; c < H * (R / 2); c += blockDim.x) {
+  for (int c = threadIdx.x; c < hn * (R / 2); c += blockDim.x) {
     const int h = c / (R / 2), i = c - h * (R / 2);
-    const T* src = q + (size_t)t * ldq + h * (D + R) + D;
+    const T* src = q + (size_t)t * ldq + (h0 + h) * (D + R) + D;
     float u = MxElem<T>::ld(src + 2 * i);
     float w = MxElem<T>::ld(src + 2 * i + 1);
     if (2 * i < rot_dims) mx_turn(u, w, cs + 2 * i, &u, &w);
-    T* dst = qf + (size_t)t * H * QW + h * QW + L;
+    T* dst = qrow + h * QW + L;
     MxElem<T>::st(dst + 2 * i, u);
     MxElem<T>::st(dst + 2 * i + 1, w);
   }
   if (R & 1)
-    for (int h = threadIdx.x; h < H; h += blockDim.x)
-      qf[(size_t)t * H * QW + h * QW + QW - 1] =
-          q[(size_t)t * ldq + h * (D + R) + D + R - 1];
+    for (int h = threadIdx.x; h < hn; h += blockDim.x)
+      qrow[h * QW + QW - 1] =
+          q[(size_t)t * ldq + (h0 + h) * (D + R) + D + R - 1];
 }
 
 // y[t] = x[t] / sqrt(mean(x[t]^2) + eps) * w. One workgroup per row.
@@ -444,14 +461,24 @@ void mx_latent_prep(void* qf, const void* qlat, const void* q, int ldq,
                     void* stream) {
   if (T_ <= 0) return;
   (void)BS;
+  dim3 grid(T_, 1 + (H + LP_HG - 1) / LP_HG);
+#define LP_GO(VEC)                                                           \
+  hipLaunchKernelGGL((latent_prep_kernel<T, VEC>), grid, dim3(256), 0,       \
+                     (hipStream_t)stream, (T*)qf, (const T*)qlat,            \
+                     (const T*)q, ldq, (const T*)dkv, lddkv,                 \
+                     (const float*)normw, eps, (const float*)cos_sin,        \
+                     table_rows, rot_dims, (const int*)positions, (T*)cache, \
+                     (const int64_t*)slots, T_, H, D, R, L)
   MX_DISPATCH_DTYPE(dtype, {
-    hipLaunchKernelGGL((latent_prep_kernel<T>), dim3(T_), dim3(256), 0,
-                       (hipStream_t)stream, (T*)qf, (const T*)qlat,
-                       (const T*)q, ldq, (const T*)dkv, lddkv,
-                       (const float*)normw, eps, (const float*)cos_sin,
-                       table_rows, rot_dims, (const int*)positions,
-                       (T*)cache, (const int64_t*)slots, T_, H, D, R, L, BS);
+    constexpr int V = 16 / sizeof(T);
+    const bool vec = L % V == 0 && (L + R) % V == 0 &&
+                     (((size_t)qf | (size_t)qlat) & 15) == 0;
+    if (vec)
+      LP_GO(true);
+    else
+      LP_GO(false);
   })
+#undef LP_GO
 }
 
 void mx_rms_norm_rows(void* y, const void* x, int ldx, const void* w,

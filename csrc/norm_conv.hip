@@ -44,11 +44,14 @@ PS_DEV void nc_st4(mx_bf16* p, const float4& v) {
 }
 
 // TD: element type of the deltas, TO: of the normed output. One workgroup
-// per row. VEC: the row is a multiple of four entries wide, at most 1024 *
-// NC_Q entries, and all rows start 16-byte aligned: a thread then keeps its
-// entries (four at a time) in registers between the passes.
+// of BT threads per row. VEC: the row is a multiple of four entries wide, at
+// most 1024 * NC_Q entries, and all rows start 16-byte aligned: a thread then
+// keeps its entries (four at a time) in registers between the passes. Steps
+// of few rows take 1024 threads per row: they do not fill the chip, so a
+// row's time is that of its chain of memory round trips.
 #define NC_Q 8
 #define NC_MAX_TAPS 32
+#define NC_SHORT 4  // taps held in registers by single-row segments
 
 // Options of the EXT form; pointers are nullptr where an option is off.
 template <typename TO>
@@ -71,6 +74,44 @@ PS_DEV void nc_single(const float* __restrict__ cw, float* __restrict__ state,
                       const float* y, float* acc) {
   const bool past = sr[2] > 0;
   float* st = state + (size_t)sr[3] * (K - 1) * W + c;
+  if (K <= NC_SHORT) {
+    // every load ahead of the first store
+    float o[NC_SHORT - 1][N], wk[NC_SHORT][N];
+    if (K == 4) {
+      // a channel's taps are one 16-byte vector
+#pragma unroll
+      for (int i = 0; i < N; ++i) {
+        const float4 q = *(const float4*)(cw + (size_t)(c + i) * 4);
+        wk[0][i] = q.x;
+        wk[1][i] = q.y;
+        wk[2][i] = q.z;
+        wk[3][i] = q.w;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < NC_SHORT; ++j)
+        if (j < K)
+#pragma unroll
+          for (int i = 0; i < N; ++i) wk[j][i] = cw[(size_t)(c + i) * K + j];
+    }
+#pragma unroll
+    for (int j = 0; j < NC_SHORT - 1; ++j)
+      if (j < K - 1)
+#pragma unroll
+        for (int i = 0; i < N; ++i)
+          o[j][i] = past ? st[(size_t)j * W + i] : 0.f;
+#pragma unroll
+    for (int j = 0; j < NC_SHORT; ++j)
+      if (j < K) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+          const float v = j < K - 1 && j < NC_SHORT - 1 ? o[j][i] : y[i];
+          acc[i] += wk[j][i] * v;
+          if (j > 0) st[(size_t)(j - 1) * W + i] = v;
+        }
+      }
+    return;
+  }
   float old[N];
 #pragma unroll
   for (int i = 0; i < N; ++i) acc[i] += cw[(size_t)(c + i) * K + K - 1] * y[i];
@@ -88,8 +129,8 @@ PS_DEV void nc_single(const float* __restrict__ cw, float* __restrict__ state,
     for (int i = 0; i < N; ++i) st[(size_t)(K - 2) * W + i] = y[i];
 }
 
-template <typename TD, typename TO, bool VEC, bool EXT>
-__global__ __launch_bounds__(256) void add_layer_norm32_kernel(
+template <typename TD, typename TO, bool VEC, bool EXT, int BT>
+__global__ __launch_bounds__(BT) void add_layer_norm32_kernel(
     TO* __restrict__ h, float* __restrict__ x, const TD* __restrict__ d0,
     int ld0, float s0, const TD* __restrict__ d1, int ld1, float s1,
     const float* __restrict__ w, const float* __restrict__ b, float eps,
@@ -98,11 +139,12 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
   const int t = blockIdx.x;
   float* xr = x + (size_t)t * W;
   if (VEC) {
-    float4 v[NC_Q];
+    constexpr int NQ = NC_Q * 256 / BT;
+    float4 v[NQ];
     float sum = 0.f;
 #pragma unroll
-    for (int i = 0; i < NC_Q; ++i) {
-      const int c = (threadIdx.x + 256 * i) * 4;
+    for (int i = 0; i < NQ; ++i) {
+      const int c = (threadIdx.x + BT * i) * 4;
       if (c < W) {
         v[i] = nc_ld4(xr + c);
         if (d0 != nullptr) {
@@ -134,8 +176,8 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
     const float mean = mx_block_sum(sum, red) / (float)W;
     float sq = 0.f;
 #pragma unroll
-    for (int i = 0; i < NC_Q; ++i) {
-      const int c = (threadIdx.x + 256 * i) * 4;
+    for (int i = 0; i < NQ; ++i) {
+      const int c = (threadIdx.x + BT * i) * 4;
       if (c < W) {
         const float e0 = v[i].x - mean, e1 = v[i].y - mean;
         const float e2 = v[i].z - mean, e3 = v[i].w - mean;
@@ -149,8 +191,8 @@ __global__ __launch_bounds__(256) void add_layer_norm32_kernel(
     }
     if (h != nullptr) {
 #pragma unroll
-      for (int i = 0; i < NC_Q; ++i) {
-        const int c = (threadIdx.x + 256 * i) * 4;
+      for (int i = 0; i < NQ; ++i) {
+        const int c = (threadIdx.x + BT * i) * 4;
         if (c < W) {
           const float4 ww = nc_ld4(w + c), bb = nc_ld4(b + c);
           float4 o;
@@ -307,11 +349,14 @@ int mx_add_layer_norm32(void* h, void* x, const void* d0, int ld0, float s0,
       W % 4 == 0 && W <= 1024 * NC_Q && ld0 % 4 == 0 && ld1 % 4 == 0 &&
       ldz % 4 == 0 &&
       (((size_t)h | (size_t)x | (size_t)d0 | (size_t)d1 | (size_t)w |
-        (size_t)b | (size_t)z | (size_t)zb | (size_t)yp) & 15) == 0;
+        (size_t)b | (size_t)z | (size_t)zb | (size_t)yp | (size_t)cw) & 15) ==
+      0;
   const bool e = z != nullptr || cw != nullptr;
-#define ALN_K(TD, TO, VEC, EXT)                                              \
-  hipLaunchKernelGGL((add_layer_norm32_kernel<TD, TO, VEC, EXT>), dim3(T_),  \
-                     dim3(256), 0, (hipStream_t)stream, (TO*)h, (float*)x,   \
+  const bool few = T_ <= 512 && W >= 2048;
+#define ALN_K(TD, TO, VEC, EXT, BT)                                          \
+  hipLaunchKernelGGL((add_layer_norm32_kernel<TD, TO, VEC, EXT, BT>),        \
+                     dim3(T_), dim3(BT), 0, (hipStream_t)stream, (TO*)h,     \
+                     (float*)x,                                              \
                      (const TD*)d0, ld0, s0, (const TD*)d1, ld1, s1,         \
                      (const float*)w, (const float*)b, eps, (float*)stats,   \
                      W,                                                      \
@@ -319,14 +364,18 @@ int mx_add_layer_norm32(void* h, void* x, const void* d0, int ld0, float s0,
                                 (TO*)yp, (const float*)cw, (float*)state,    \
                                 (const int*)seq_rows, K}))
 #define ALN_GO(TD, TO)                                                       \
-  if (vec && e)                                                              \
-    ALN_K(TD, TO, true, true);                                               \
+  if (vec && few && e)                                                       \
+    ALN_K(TD, TO, true, true, 1024);                                         \
+  else if (vec && few)                                                       \
+    ALN_K(TD, TO, true, false, 1024);                                        \
+  else if (vec && e)                                                         \
+    ALN_K(TD, TO, true, true, 256);                                          \
   else if (vec)                                                              \
-    ALN_K(TD, TO, true, false);                                              \
+    ALN_K(TD, TO, true, false, 256);                                         \
   else if (e)                                                                \
-    ALN_K(TD, TO, false, true);                                              \
+    ALN_K(TD, TO, false, true, 256);                                         \
   else                                                                       \
-    ALN_K(TD, TO, false, false)
+    ALN_K(TD, TO, false, false, 256)
   if (delta_dtype == MX_BF16) {
     if (out_dtype == MX_BF16) {
       ALN_GO(mx_bf16, mx_bf16);
