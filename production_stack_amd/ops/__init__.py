@@ -641,7 +641,9 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     both falling back to the plain one-workgroup-per-token kernel; 1 / 2 /
     4 force plain / tiled / split-key. bfloat16 batches without head mix
     and aligned chunks take the matrix-core kernel instead when the shape
-    fits it (variants 0 and 3; 5 insists on it, 6 on its 128-row form).
+    fits it (variants 0 and 3; 5 insists on it, 6 on its 128-row form);
+    single tokens over rows that carry their values take a kernel of their
+    own first (variant 3; 7 insists on it).
     Returns [T, H*DV]."""
     NB, G, BS, D = k_cache.shape
     VR = v_cache.shape[3]
@@ -689,6 +691,24 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     # workgroup per token, each token's keys are shared out over several
     # workgroups whose partial softmax records are merged afterwards
     scratch = None
+    if (variant in (3, 7) and q.dtype == torch.bfloat16 and G == 1
+            and v_cache.data_ptr() == k_cache.data_ptr() and talk is None
+            and chunk == 0 and keep_first == 0 and softcap == 0.0):
+        shares = splits if splits > 0 else max(
+            1, min(16 if T <= 4 else 8, 256 // (T * ((H + 31) // 32))))
+        part = (torch.empty((T, shares, H, DV + 4), dtype=torch.float32,
+                            device=q.device) if shares > 1 else None)
+        rc = _mx().mx_latent_decode(
+            _p(out), _rows(out, "out"), _p(q), _rows(q, "q"), _p(k_cache),
+            _p(block_tables), block_tables.shape[1], _p(token_seq),
+            _p(token_pos), T, H, D, DV, BS, _f(scale), int(window),
+            int(bool(sink)), _p(sink_vals), int(shares), _p(part),
+            _stream())
+        if rc == 0:
+            return out
+    if variant == 7:
+        raise RuntimeError(
+            "talk_attention: shape or dtype outside the latent-row kernel")
     if variant not in (3, 4, 5, 6):
         splits = 1
     elif splits <= 0:

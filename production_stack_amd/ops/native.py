@@ -10,8 +10,8 @@ shape checks live in the Python wrappers
 
 Groups (one shared library each):
   core    resid32, norm_conv, mixer_prep, talk_attention, mfma_attention,
-          expand_attention, moe_route, moe_group, mingru_scan
-                                            -> _mixops.so
+          expand_attention, latent_decode, moe_route, moe_group,
+          mingru_scan                       -> _mixops.so
   delta   delta_rule                        -> _mixops_delta.so
   gdelta  gated_delta                       -> _mixops_gdelta.so
   scan    linear_scan                       -> _mixops_scan.so
@@ -47,6 +47,7 @@ GROUPS = {
         ("mixer_prep.hip", []),
         ("mfma_attention.hip", []),
         ("expand_attention.hip", []),
+        ("latent_decode.hip", []),
         ("moe_route.hip", []),
         ("moe_group.hip", []),
         ("mingru_scan.hip", []),
@@ -84,6 +85,7 @@ INT_RESULT = {
     "mx_short_conv_silu", "mx_mfma_attention", "mx_linear_scan",
     "mx_linear_scan_splits", "mx_norm_conv32", "mx_moe_route",
     "mx_add_layer_norm32", "mx_expert_plan", "mx_expand_attention",
+    "mx_latent_decode",
 }
 
 # entry points that return a 64-bit count

@@ -499,6 +499,52 @@ def test_expanded_attention_kernel(shape):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("shape", [
+    # heads, row, value columns, window, sink, page
+    (32, 576, 512, 0, None, 16), (3, 72, 40, 50, None, 16),
+    (1, 24, 16, 1, None, 16), (32, 288, 256, 129, "learned", 16),
+    (40, 128, 100, 64, "zero", 7), (64, 320, 256, 200, None, 32),
+    (5, 296, 290, 65, "learned", 16)])
+@pytest.mark.parametrize("splits", [0, 1, 3, 8])
+def test_latent_decode_kernel(shape, splits):
+    """Single tokens over latent rows: lengths around tile borders, shares
+    with and without keys, a key that stands out just inside and outside
+    the window, on a page border and at the start."""
+    H, D, DV, win, sink, BS = shape
+    bf = torch.bfloat16
+    lens = [1, 2, 63, 64, 65, 200, 129, 5, 400]
+    S, per = len(lens), 400 // BS + 1
+    g = torch.Generator().manual_seed(H + D)
+    tables = torch.randperm(S * per + 3, generator=g)[:S * per].view(
+        S, per).int()
+    cache = rnd((S * per + 3, 1, BS, D), 1, 1.0, bf)
+    q = rnd((S, H * D + 8), 2, 0.5, bf)[:, 8:]
+    sv = rnd((H,), 5) if sink == "learned" else None
+    pos = torch.tensor([n - 1 for n in lens], dtype=torch.int32)
+    seq = torch.arange(S, dtype=torch.int32)
+    for back in [None, 0, BS, max(win, 1) - 1, max(win, 1), 399]:
+        c = cache.clone()
+        if back is not None:       # every head of a token likes this key
+            for s, n in enumerate(lens):
+                j = n - 1 - back
+                if j >= 0:
+                    c[tables[s, j // BS], 0, j % BS] = \
+                        q[s].view(H, D).float().mean(0).to(bf) * 6
+        kw = dict(window=win, sink=bool(sink), vdim=DV)
+        want = R.talk_attention(
+            q.reshape(S, H, D), c, c, tables, seq, pos, D ** -0.5, 0, win,
+            bool(sink), None, 0, 0.0, sv, DV).reshape(S, H * DV)
+        cc = c.cuda()
+        got = ops.talk_attention(
+            q.cuda(), cc, cc, tables.cuda(), seq.cuda(), pos.cuda(),
+            D ** -0.5, H, variant=7, splits=splits,
+            sink_vals=sv.cuda() if sv is not None else None, **kw)
+        err = (got.cpu().float() - want.float()).norm(dim=-1) / \
+            want.float().norm(dim=-1)
+        assert float(err.max()) < 1e-2, back
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("act,gated", [("silu", True), ("gelu_tanh", True),
                                        ("clamped_swish", True),
                                        ("relu2", False), ("silu", False)])
