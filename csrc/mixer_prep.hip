@@ -2,6 +2,9 @@
 //   attn_prep        per-head query/key RMSNorm, rotary turn of the heads'
 //                    leading entries, value blend with another layer's
 //                    values, paged K/V append;
+//   keyval_prep      queries over their root mean square per head, paged
+//                    append of keys that are also the values, with one over
+//                    their root mean square beside them;
 //   latent_prep      latent RMSNorm, rotary turn of the shared key part and
 //                    of the queries' rotary parts, paged append of
 //                    [latent | key part], assembly of the latent-space
@@ -185,6 +188,65 @@ __global__ __launch_bounds__(256) void pool_append_kernel(
   MxElem<T>::st((is_k ? kp : vp) + prow * w + d, acc / (float)pool);
 }
 
+// Queries and keys of attention whose keys are their own values. A group of
+// `lanes` lanes (a power of two) takes one head: a query head is divided by
+// its root mean square in place, a key head goes to its cache row as it is and
+// its 1/rms to kscale [NB, G, BS]. V entries per access; the first one of a
+// lane stays in registers between the passes.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void keyval_prep_kernel(
+    T* __restrict__ q, int ldq, const T* __restrict__ k, int ldk, float eps,
+    T* __restrict__ cache, float* __restrict__ kscale,
+    const int64_t* __restrict__ slots, int H, int G, int D, int BS,
+    int lanes) {
+  struct __align__(sizeof(T) * V) Vec {
+    T e[V];
+  };
+  const int t = blockIdx.x;
+  const int64_t slot = slots[t];
+  const int per = blockDim.x / lanes;
+  const int gl = threadIdx.x & (lanes - 1), nv = D / V;
+  for (int h0 = 0; h0 < H + G; h0 += per) {
+    // every lane joins the exchanges below; idle groups repeat the last head
+    const int hh = h0 + threadIdx.x / lanes;
+    const int hc = min(hh, H + G - 1);
+    const bool is_q = hc < H;
+    const T* src = is_q ? q + (size_t)t * ldq + (size_t)hc * D
+                        : k + (size_t)t * ldk + (size_t)(hc - H) * D;
+    float ss = 0.f;
+    Vec first;
+    for (int c = gl; c < nv; c += lanes) {
+      const Vec v = *(const Vec*)(src + c * V);
+      if (c == gl) first = v;
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        const float x = MxElem<T>::ld(&v.e[i]);
+        ss += x * x;
+      }
+    }
+    for (int off = lanes >> 1; off > 0; off >>= 1)
+      ss += __shfl_xor(ss, off, 64);
+    const float inv = 1.0f / sqrtf(ss / (float)D + eps);
+    if (hh >= H + G) continue;
+    if (is_q) {
+      T* dst = q + (size_t)t * ldq + (size_t)hc * D;
+      for (int c = gl; c < nv; c += lanes) {
+        Vec v = c == gl ? first : *(const Vec*)(src + c * V);
+#pragma unroll
+        for (int i = 0; i < V; ++i)
+          MxElem<T>::st(&v.e[i], MxElem<T>::ld(&v.e[i]) * inv);
+        *(Vec*)(dst + c * V) = v;
+      }
+    } else if (slot >= 0) {
+      const int64_t row = ((slot / BS) * G + (hc - H)) * BS + slot % BS;
+      T* dst = cache + row * D;
+      for (int c = gl; c < nv; c += lanes)
+        *(Vec*)(dst + c * V) = c == gl ? first : *(const Vec*)(src + c * V);
+      if (gl == 0) kscale[row] = inv;
+    }
+  }
+}
+
 // Turn the pair (u, w) by the table entry (cos, sin).
 PS_DEV void mx_turn(float u, float w, const float* cs, float* ou, float* ow) {
   *ou = u * cs[0] - w * cs[1];
@@ -192,9 +254,20 @@ PS_DEV void mx_turn(float u, float w, const float* cs, float* ou, float* ow) {
 }
 
 // Grid (tokens, 1 + head groups): workgroup y = 0 normalises the latent,
-// turns the shared key part and appends the row; workgroup y > 0 assembles
-// the queries of HG heads. VEC: latent parts are whole 16-byte vectors.
+// turns the shared key part and appends the row (nothing to do without dkv:
+// the rows are another layer's); workgroup y > 0 assembles the queries of HG
+// heads. VEC: latent parts are whole 16-byte vectors. half: the rotary pairs
+// are (i, i + rot_dims / 2) instead of neighbours.
 #define LP_HG 4
+
+// Entries of pair i of a rotary part of R entries: pairs below rot_dims / 2
+// turn; the rest (every pair that lies past rot_dims) passes.
+PS_DEV void lp_pair(int i, int rot_dims, int half, int* a, int* b) {
+  const int hd = rot_dims >> 1;
+  const bool split = half && i < hd;
+  *a = split ? i : 2 * i;
+  *b = split ? i + hd : 2 * i + 1;
+}
 
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void latent_prep_kernel(
@@ -202,12 +275,14 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     const T* __restrict__ dkv, int lddkv, const float* __restrict__ normw,
     float eps, const float* __restrict__ cos_sin, int table_rows,
     int rot_dims, const int* __restrict__ positions, T* __restrict__ cache,
-    const int64_t* __restrict__ slots, int T_, int H, int D, int R, int L) {
+    const int64_t* __restrict__ slots, int T_, int H, int D, int R, int L,
+    int half) {
   __shared__ float red[17];
   const int t = blockIdx.x;
   const int pos = min(max(positions[t], 0), table_rows - 1);
   const float* cs = cos_sin + (size_t)pos * rot_dims;  // [rot_dims/2][2]
   if (blockIdx.y == 0) {
+    if (dkv == nullptr) return;
     const T* row = dkv + (size_t)t * lddkv;
     const int64_t slot = slots[t];
     T* crow = cache + (slot >= 0 ? slot : 0) * (int64_t)(L + R);
@@ -223,11 +298,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
       MxElem<T>::st(crow + c, MxElem<T>::ld(row + c) * inv * normw[c]);
     // shared key part: pairs below rot_dims turn, the rest passes
     for (int i = threadIdx.x; i < R / 2; i += blockDim.x) {
-      float u = MxElem<T>::ld(row + L + 2 * i);
-      float w = MxElem<T>::ld(row + L + 2 * i + 1);
+      int a, b;
+      lp_pair(i, rot_dims, half, &a, &b);
+      float u = MxElem<T>::ld(row + L + a);
+      float w = MxElem<T>::ld(row + L + b);
       if (2 * i < rot_dims) mx_turn(u, w, cs + 2 * i, &u, &w);
-      MxElem<T>::st(crow + L + 2 * i, u);
-      MxElem<T>::st(crow + L + 2 * i + 1, w);
+      MxElem<T>::st(crow + L + a, u);
+      MxElem<T>::st(crow + L + b, w);
     }
     if ((R & 1) && threadIdx.x == 0) crow[L + R - 1] = row[L + R - 1];
     return;
@@ -238,11 +315,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     // a thread owns both entries of a pair
     for (int c = threadIdx.x; c < hn * (rot_dims / 2); c += blockDim.x) {
       const int h = c / (rot_dims / 2), i = c - h * (rot_dims / 2);
-      T* p = qf + (size_t)t * ldq + (h0 + h) * (D + R) + D + 2 * i;
+      T* p = qf + (size_t)t * ldq + (h0 + h) * (D + R) + D;
+      int a, b;
+      lp_pair(i, rot_dims, half, &a, &b);
       float u, w;
-      mx_turn(MxElem<T>::ld(p), MxElem<T>::ld(p + 1), cs + 2 * i, &u, &w);
-      MxElem<T>::st(p, u);
-      MxElem<T>::st(p + 1, w);
+      mx_turn(MxElem<T>::ld(p + a), MxElem<T>::ld(p + b), cs + 2 * i, &u, &w);
+      MxElem<T>::st(p + a, u);
+      MxElem<T>::st(p + b, w);
     }
     return;
   }
@@ -266,12 +345,14 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
   for (int c = threadIdx.x; c < hn * (R / 2); c += blockDim.x) {
     const int h = c / (R / 2), i = c - h * (R / 2);
     const T* src = q + (size_t)t * ldq + (h0 + h) * (D + R) + D;
-    float u = MxElem<T>::ld(src + 2 * i);
-    float w = MxElem<T>::ld(src + 2 * i + 1);
+    int a, b;
+    lp_pair(i, rot_dims, half, &a, &b);
+    float u = MxElem<T>::ld(src + a);
+    float w = MxElem<T>::ld(src + b);
     if (2 * i < rot_dims) mx_turn(u, w, cs + 2 * i, &u, &w);
     T* dst = qrow + h * QW + L;
-    MxElem<T>::st(dst + 2 * i, u);
-    MxElem<T>::st(dst + 2 * i + 1, w);
+    MxElem<T>::st(dst + a, u);
+    MxElem<T>::st(dst + b, w);
   }
   if (R & 1)
     for (int h = threadIdx.x; h < hn; h += blockDim.x)
@@ -436,6 +517,30 @@ void mx_attn_prep(void* q, int ldq, const void* k, int ldk, void* v, int ldv,
 #undef AP_GO
 }
 
+void mx_keyval_prep(void* q, int ldq, const void* k, int ldk, float eps,
+                    void* cache, void* kscale, const void* slots, int T_,
+                    int H, int G, int D, int BS, int dtype, void* stream) {
+  if (T_ <= 0 || H <= 0 || G <= 0 || D <= 0) return;
+  const bool aligned = (((size_t)q | (size_t)k | (size_t)cache) & 15) == 0;
+#define KP_GO(V)                                                             \
+  {                                                                          \
+    int lanes = 1;                                                           \
+    while (lanes < 64 && lanes * (V) < D) lanes <<= 1;                       \
+    hipLaunchKernelGGL((keyval_prep_kernel<T, V>), dim3(T_), dim3(256), 0,   \
+                       (hipStream_t)stream, (T*)q, ldq, (const T*)k, ldk,    \
+                       eps, (T*)cache, (float*)kscale,                       \
+                       (const int64_t*)slots, H, G, D, BS, lanes);           \
+  }
+  MX_DISPATCH_DTYPE(dtype, {
+    constexpr int VN = 16 / sizeof(T);
+    if (aligned && D % VN == 0 && ldq % VN == 0 && ldk % VN == 0)
+      KP_GO(VN)
+    else
+      KP_GO(1)
+  })
+#undef KP_GO
+}
+
 void mx_pool_append(const void* kc, const void* vc, void* kp, void* vp,
                     const void* block_tables, int max_blocks,
                     const void* seq_rows, int S_, int blocks_per_seg, int G,
@@ -457,8 +562,8 @@ void mx_latent_prep(void* qf, const void* qlat, const void* q, int ldq,
                     const void* dkv, int lddkv, const void* normw, float eps,
                     const void* cos_sin, int table_rows, int rot_dims,
                     const void* positions, void* cache, const void* slots,
-                    int T_, int H, int D, int R, int L, int BS, int dtype,
-                    void* stream) {
+                    int T_, int H, int D, int R, int L, int BS, int half,
+                    int dtype, void* stream) {
   if (T_ <= 0) return;
   (void)BS;
   dim3 grid(T_, 1 + (H + LP_HG - 1) / LP_HG);
@@ -468,7 +573,7 @@ void mx_latent_prep(void* qf, const void* qlat, const void* q, int ldq,
                      (const T*)q, ldq, (const T*)dkv, lddkv,                 \
                      (const float*)normw, eps, (const float*)cos_sin,        \
                      table_rows, rot_dims, (const int*)positions, (T*)cache, \
-                     (const int64_t*)slots, T_, H, D, R, L)
+                     (const int64_t*)slots, T_, H, D, R, L, half)
   MX_DISPATCH_DTYPE(dtype, {
     constexpr int V = 16 / sizeof(T);
     const bool vec = L % V == 0 && (L + R) % V == 0 &&

@@ -1,10 +1,11 @@
 // Router of a routed feed-forward, one kernel per layer and step:
-//   logits = W_router x            (fp32 accumulation of the inputs' products)
+//   logits = W_router x + bias     (fp32 accumulation of the inputs' products;
+//            the bias is optional)
 //   scores = softmax(logits)  |  sigmoid(logits)
 //   choice = the `top` largest of scores + correction (the correction only
-//            moves the choice); sigmoid scores without a correction are
-//            ranked by their logits (the fp32 sigmoid saturates and would
-//            tie large scores)
+//            moves the choice); scores without a correction are ranked by
+//            their logits (the fp32 sigmoid saturates and would tie large
+//            scores, the softmax underflows and would tie small ones)
 //   weights = the chosen scores, divided by (their sum + renorm_eps) when
 //            asked, times scale
 // Outputs: the chosen outputs' indices and weights [T, top] (best first) and
@@ -66,9 +67,9 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_route_kernel(
     int64_t* __restrict__ sel, float* __restrict__ wts,
     float* __restrict__ dense, const T* __restrict__ x, int ldx,
-    const T* __restrict__ rw, const float* __restrict__ corr, int T_, int W,
-    int n_out, int top, int sigmoid_scores, int renorm, float renorm_eps,
-    float scale, int vec) {
+    const T* __restrict__ rw, const float* __restrict__ corr,
+    const float* __restrict__ bias, int T_, int W, int n_out, int top,
+    int sigmoid_scores, int renorm, float renorm_eps, float scale, int vec) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int nw = blockDim.x >> 6;
@@ -80,7 +81,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   for (int e = wave; e < n_out; e += nw) {
     const float acc =
         mx_wave_sum(mr_dot(xr, rw + (size_t)e * W, W, lane, vec != 0));
-    if (lane == 0) score[e] = acc;
+    if (lane == 0) score[e] = bias != nullptr ? acc + bias[e] : acc;
   }
   __syncthreads();
   if (wave != 0) return;  // the rest is one wave's work
@@ -99,9 +100,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     for (int e = lane; e < n_out; e += 64) s += expf(score[e] - m);
     s = mx_wave_sum(s);
     for (int e = lane; e < n_out; e += 64) {
-      const float p = expf(score[e] - m) / s;
+      const float z = score[e];
+      const float p = expf(z - m) / s;
       score[e] = p;
-      pick[e] = corr != nullptr ? p + corr[e] : p;
+      pick[e] = corr != nullptr ? p + corr[e] : z;
     }
   }
   __builtin_amdgcn_wave_barrier();
@@ -193,10 +195,11 @@ extern "C" void mx_moe_combine(void* out, const void* y, const void* dense,
 }
 
 extern "C" int mx_moe_route(void* sel, void* wts, void* dense, const void* x,
-                            int ldx, const void* rw, const void* corr, int T_,
-                            int W, int n_out, int top, int sigmoid_scores,
-                            int renorm, float renorm_eps, float scale,
-                            int dtype, void* stream) {
+                            int ldx, const void* rw, const void* corr,
+                            const void* bias, int T_, int W, int n_out,
+                            int top, int sigmoid_scores, int renorm,
+                            float renorm_eps, float scale, int dtype,
+                            void* stream) {
   if (T_ <= 0) return 0;
   if (n_out < 1 || n_out > MR_MAX_OUT || top < 1 || top > n_out) return 1;
   const size_t lds = (size_t)(2 * n_out + top) * sizeof(float);
@@ -210,8 +213,8 @@ extern "C" int mx_moe_route(void* sel, void* wts, void* dense, const void* x,
     hipLaunchKernelGGL((moe_route_kernel<T>), dim3(T_), dim3(256), lds,
                        (hipStream_t)stream, (int64_t*)sel, (float*)wts,
                        (float*)dense, (const T*)x, ldx, (const T*)rw,
-                       (const float*)corr, T_, W, n_out, top, sigmoid_scores,
-                       renorm, renorm_eps, scale, vec);
+                       (const float*)corr, (const float*)bias, T_, W, n_out,
+                       top, sigmoid_scores, renorm, renorm_eps, scale, vec);
   })
   return 0;
 }

@@ -365,11 +365,36 @@ __global__ __launch_bounds__(256) void norm_sum32_kernel(
 
 // Sublayer boundary of a stack that normalises a sublayer's output before it
 // joins the stream: x[t] += d[t] / rms(d[t]) * wpost, then
-// h[t] = x[t] / rms(x[t]) * wnext. TD is the element type of the sublayer
-// output (fp32 for fp32 sums of experts), T of the next sublayer's input.
-// Every thread revisits the entries it wrote itself.
-template <typename TD, typename T>
-__global__ __launch_bounds__(256) void post_norm_add_norm32_kernel(
+// h[t] = x[t] / rms(x[t]) * wnext, or x[t] itself where wnext is nullptr. TD is
+// the element type of the sublayer output (fp32 for fp32 sums of experts), T of
+// the next sublayer's input. One workgroup of BT threads per row. VEC: the row
+// is a multiple of four entries wide, at most 4 BT PN_ROW, and all rows start
+// on 16 (bf16: 8) bytes: a thread then keeps its entries in registers between
+// the passes, and the stream's are on their way while the first sum is formed.
+// Otherwise every thread revisits the entries it wrote itself.
+#define PN_ROW 8
+
+PS_DEV float4 pn_ld4(const float* p) { return *(const float4*)p; }
+PS_DEV float4 pn_ld4(const mx_bf16* p) {
+  const uint2 u = *(const uint2*)p;
+  return make_float4(__uint_as_float(u.x << 16),
+                     __uint_as_float(u.x & 0xffff0000u),
+                     __uint_as_float(u.y << 16),
+                     __uint_as_float(u.y & 0xffff0000u));
+}
+PS_DEV void pn_st4(float* p, const float4& v) { *(float4*)p = v; }
+PS_DEV void pn_st4(mx_bf16* p, const float4& v) {
+  *(uint2*)p = make_uint2((unsigned int)ps_f32_to_bf16(v.x) |
+                              ((unsigned int)ps_f32_to_bf16(v.y) << 16),
+                          (unsigned int)ps_f32_to_bf16(v.z) |
+                              ((unsigned int)ps_f32_to_bf16(v.w) << 16));
+}
+PS_DEV float pn_sq(const float4& v) {
+  return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+}
+
+template <typename TD, typename T, bool VEC, int BT>
+__global__ __launch_bounds__(BT) void post_norm_add_norm32_kernel(
     T* __restrict__ h, float* __restrict__ x, const TD* __restrict__ d,
     int ldd, const float* __restrict__ wpost, const float* __restrict__ wnext,
     float eps, int W) {
@@ -377,23 +402,94 @@ __global__ __launch_bounds__(256) void post_norm_add_norm32_kernel(
   const int t = blockIdx.x;
   const TD* dr = d + (size_t)t * ldd;
   float* xr = x + (size_t)t * W;
-  float ss = 0.f;
-  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+  T* hr = h + (size_t)t * W;
+  float ss = 0.f, sx = 0.f;
+  if (VEC) {
+    float4 dv[PN_ROW], xv[PN_ROW];
+#pragma unroll
+    for (int i = 0; i < PN_ROW; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      if (c < W) {
+        dv[i] = pn_ld4(dr + c);
+        xv[i] = pn_ld4(xr + c);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < PN_ROW; ++i)
+      if (4 * (threadIdx.x + BT * i) < W) ss += pn_sq(dv[i]);
+    ss = mx_block_sum(ss, red);
+    const float dinv = 1.0f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < PN_ROW; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      if (c < W) {
+        const float4 w = pn_ld4(wpost + c);
+        xv[i].x += dv[i].x * dinv * w.x;
+        xv[i].y += dv[i].y * dinv * w.y;
+        xv[i].z += dv[i].z * dinv * w.z;
+        xv[i].w += dv[i].w * dinv * w.w;
+        pn_st4(xr + c, xv[i]);
+        if (wnext == nullptr)
+          pn_st4(hr + c, xv[i]);
+        else
+          sx += pn_sq(xv[i]);
+      }
+    }
+    if (wnext == nullptr) return;
+    sx = mx_block_sum(sx, red);
+    const float xinv = 1.0f / sqrtf(sx / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < PN_ROW; ++i) {
+      const int c = 4 * (threadIdx.x + BT * i);
+      if (c < W) {
+        const float4 w = pn_ld4(wnext + c);
+        pn_st4(hr + c,
+               make_float4(xv[i].x * xinv * w.x, xv[i].y * xinv * w.y,
+                           xv[i].z * xinv * w.z, xv[i].w * xinv * w.w));
+      }
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < W; c += BT) {
     const float v = MxElem<TD>::ld(dr + c);
     ss += v * v;
   }
   ss = mx_block_sum(ss, red);
   const float dinv = 1.0f / sqrtf(ss / (float)W + eps);
-  float sx = 0.f;
-  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+  for (int c = threadIdx.x; c < W; c += BT) {
     const float v = xr[c] + MxElem<TD>::ld(dr + c) * dinv * wpost[c];
     xr[c] = v;
+    if (wnext == nullptr) MxElem<T>::st(hr + c, v);
     sx += v * v;
   }
+  if (wnext == nullptr) return;
   sx = mx_block_sum(sx, red);
   const float xinv = 1.0f / sqrtf(sx / (float)W + eps);
-  for (int c = threadIdx.x; c < W; c += blockDim.x)
-    MxElem<T>::st(h + (size_t)t * W + c, xr[c] * xinv * wnext[c]);
+  for (int c = threadIdx.x; c < W; c += BT)
+    MxElem<T>::st(hr + c, xr[c] * xinv * wnext[c]);
+}
+
+// Steps of few rows take 1024 threads per row: they do not fill the chip, so a
+// row's time is that of its chain of memory round trips.
+template <typename TD, typename T>
+static void pn_launch(void* h, void* x, const void* d, int ldd,
+                      const void* wpost, const void* wnext, float eps, int T_,
+                      int W, hipStream_t stream) {
+  const bool vec =
+      W % 4 == 0 && ldd % 4 == 0 && W <= 4 * 256 * PN_ROW &&
+      (((size_t)h | (size_t)x | (size_t)d | (size_t)wpost | (size_t)wnext) &
+       15) == 0;
+#define PN_GO(VEC, BT)                                                       \
+  hipLaunchKernelGGL((post_norm_add_norm32_kernel<TD, T, VEC, BT>), dim3(T_), \
+                     dim3(BT), 0, stream, (T*)h, (float*)x, (const TD*)d,    \
+                     ldd, (const float*)wpost, (const float*)wnext, eps, W)
+  if (!vec)
+    PN_GO(false, 256);
+  else if (T_ <= 256 && W > 1024)
+    PN_GO(true, 1024);
+  else
+    PN_GO(true, 256);
+#undef PN_GO
 }
 
 extern "C" {
@@ -572,17 +668,12 @@ void mx_post_norm_add_norm32(void* h, void* x, const void* d, int ldd,
                              int dtype, void* stream) {
   if (T_ <= 0) return;
   MX_DISPATCH_DTYPE(dtype, {
-    if (d_dtype == MX_BF16) {
-      hipLaunchKernelGGL((post_norm_add_norm32_kernel<mx_bf16, T>), dim3(T_),
-                         dim3(256), 0, (hipStream_t)stream, (T*)h, (float*)x,
-                         (const mx_bf16*)d, ldd, (const float*)wpost,
-                         (const float*)wnext, eps, W);
-    } else {
-      hipLaunchKernelGGL((post_norm_add_norm32_kernel<float, T>), dim3(T_),
-                         dim3(256), 0, (hipStream_t)stream, (T*)h, (float*)x,
-                         (const float*)d, ldd, (const float*)wpost,
-                         (const float*)wnext, eps, W);
-    }
+    if (d_dtype == MX_BF16)
+      pn_launch<mx_bf16, T>(h, x, d, ldd, wpost, wnext, eps, T_, W,
+                            (hipStream_t)stream);
+    else
+      pn_launch<float, T>(h, x, d, ldd, wpost, wnext, eps, T_, W,
+                          (hipStream_t)stream);
   })
 }
 

@@ -10,6 +10,11 @@
 // its first position at row (first position mod BS) div pool of a pooled
 // cache with ceil(BS / pool) rows per page. The kernels walk three key
 // ranges in turn: kept first keys, pooled blocks, window.
+// Without pooled blocks a key's scores can carry a factor of their own
+// (TaOpt::kscale, fp32 [NB, G, BS]: one over the root mean square of a key
+// that is cached as projected because it is also the value), and a linear
+// penalty slope_h * (query position - key position) can be taken off
+// (TaOpt::slopes).
 //
 // One launch covers a ragged batch: every token carries (its sequence's
 // block-table row, its position); keys and values come from the paged
@@ -38,6 +43,8 @@ struct TaOpt {
   const void* vp;  // pooled values [NB, G, pr, DV]
   int pool;        // positions per pooled block
   int pr;          // pooled rows per page
+  const float* kscale;  // factor per cached key (nullptr: none)
+  const float* slopes;  // distance slope per head (nullptr: none)
 };
 
 // Pooled blocks a query at position pos sees behind its window.
@@ -53,6 +60,15 @@ PS_DEV int64_t ta_row(const int* __restrict__ table, int j, int G, int g,
   if (P == 1) return ((int64_t)table[j / BS] * G + g) * BS + (j % BS);
   const int pos = j * P;
   return ((int64_t)table[pos / BS] * G + g) * R + (pos % BS) / P;
+}
+
+// A scaled score with the key's factor (row: the key's row of the cache
+// [NB, G, BS]) and the distance penalty.
+PS_DEV float ta_adjust(const TaOpt& opt, float sc, int64_t row, int h,
+                       int dist) {
+  if (opt.kscale != nullptr) sc *= opt.kscale[row];
+  if (opt.slopes != nullptr) sc -= opt.slopes[h] * (float)dist;
+  return sc;
 }
 
 PS_DEV float ta_cap(float sc, float cap) {
@@ -89,6 +105,7 @@ __global__ __launch_bounds__(256) void talk_attn_kernel(
   q += h0 * D;
   out += h0 * DV;
   if (opt.sink_vals) opt.sink_vals += h0;
+  if (opt.slopes) opt.slopes += h0;
   float* sq = lds;                 // [H*D]
   float* ss = sq + H * D;          // [H][KT] raw scores
   float* sp = ss + H * TA_KT;      // [H][KT] mixed scores -> weights
@@ -133,12 +150,12 @@ __global__ __launch_bounds__(256) void talk_attn_kernel(
     for (int it = threadIdx.x; it < H * nk; it += blockDim.x) {
       const int jj = it / H, h = it % H;
       const int j = j0 + jj;
-      const T* kr =
-          kcr + ta_row(table, j, G, (h0 + h) / rep, BS, cP, cR) * (int64_t)D;
+      const int64_t krow = ta_row(table, j, G, (h0 + h) / rep, BS, cP, cR);
+      const T* kr = kcr + krow * (int64_t)D;
       const float* qh = sq + h * D;
       float acc = 0.f;
       for (int d = 0; d < D; ++d) acc += qh[d] * MxElem<T>::ld(kr + d);
-      ss[h * TA_KT + jj] = acc * scale;
+      ss[h * TA_KT + jj] = ta_adjust(opt, acc * scale, krow, h, pos - j);
     }
     __syncthreads();
     // mix across heads
@@ -399,8 +416,11 @@ __global__ __launch_bounds__(256) void talk_attn_tiled_kernel(
           } else {
             sc = sS[jj * NP + tid];
           }
-          sc = ta_cap(sc, opt.softcap);
           const int j = j0 + jj;
+          if (opt.kscale != nullptr || opt.slopes != nullptr)
+            sc = ta_adjust(opt, sc, ta_row(table, j, G, gk, BS, 1, BS), h,
+                           my_pos - j);
+          sc = ta_cap(sc, opt.softcap);
           if (rg == 1 ? j >= my_pool
                       : (j > my_pos || (j < my_lo && j >= opt.keep_first)))
             sc = PS_NEG_INF;
@@ -512,6 +532,7 @@ __global__ __launch_bounds__(256) void talk_attn_split_kernel(
   const int gk = valid ? h / rep : 0;
   const int* table = block_tables + (size_t)token_seq[t] * max_blocks;
   int lo = 0, pos = token_pos[t];
+  const int qpos = pos;
   if (chunk > 0) lo = (pos / chunk) * chunk;
   if (window > 0) lo = max(lo, pos - window + 1);
   // the kept first keys and the pooled blocks behind the window go to
@@ -594,6 +615,9 @@ __global__ __launch_bounds__(256) void talk_attn_split_kernel(
           } else {
             sc = sS[jj * H + h];
           }
+          if (opt.kscale != nullptr || opt.slopes != nullptr)
+            sc = ta_adjust(opt, sc, ta_row(table, j0 + jj, G, gk, BS, 1, BS),
+                           h, qpos - (j0 + jj));
           sc = ta_cap(sc, opt.softcap);
           const float mx = fmaxf(m, sc);
           const float alpha = expf(m - mx);  // m = -inf gives 0
@@ -761,14 +785,18 @@ extern "C" int mx_talk_attention(void* out, int ldout, const void* q,
                                  int splits, void* scratch, int keep_first,
                                  float softcap, const void* sink_vals,
                                  int vrow, const void* kpool,
-                                 const void* vpool, int pool, void* stream) {
+                                 const void* vpool, int pool,
+                                 const void* kscale, const void* slopes,
+                                 void* stream) {
   if (T_ <= 0) return 0;
   if (vrow < DV) return 3;
   const bool pooled = kpool != nullptr && pool > 0 && window > 0;
   const TaOpt opt = {keep_first > 0 ? keep_first : 0, softcap,
                      (const float*)sink_vals, vrow,
                      pooled ? kpool : nullptr, pooled ? vpool : nullptr,
-                     pooled ? pool : 0, pooled ? (BS + pool - 1) / pool : 0};
+                     pooled ? pool : 0, pooled ? (BS + pool - 1) / pool : 0,
+                     (const float*)kscale, (const float*)slopes};
+  if (pooled && (kscale != nullptr || slopes != nullptr)) return 3;
   const int dmax = D > DV ? D : DV;
   if ((variant == 0 || variant == 2) && H <= 256 && dmax <= 128) {
     int rc = 1;

@@ -76,6 +76,14 @@ class MixerSpec:
     (heads = 1) whose gate and candidate read the current token only:
     S <- (1 - z) S + z c, z = sigmoid(W_z h + b_z), c = u + 1/2 for
     u = W_x h + b_x >= 0 and sigmoid(u) below; read-out S silu(W_g h).
+    Attention options: `key_values` has no value projection, the values are
+    the projected keys before their norm; `unit_qk` divides every query and
+    key head by its root mean square (no learned weight); `distance_bias`
+    takes slope_h * (query position - key position) off the scaled scores,
+    slope_h = 2^(-8 (h + 1) / heads).
+    Latent attention: `kv_from` = j has no latent of its own and attends
+    over layer j's cached rows through up-projections of its own;
+    `rot_layout` applies to the rotated parts here too.
     """
 
     kind: str
@@ -121,6 +129,10 @@ class MixerSpec:
     right_scale: float = 1.0
     q_rank: int = 0
     head_gate: bool = False
+    key_values: bool = False
+    unit_qk: bool = False
+    distance_bias: bool = False
+    kv_from: Optional[int] = None
 
 
 @dataclass
@@ -141,7 +153,8 @@ class MlpSpec:
     `table_rows` rows gives every token id its `top` experts, each with
     weight 1 / top. act "poly_norm" (dense, not gated): with N(v) = v over
     its root mean square, c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, four learned
-    numbers."""
+    numbers. `router_bias`: a learned offset joins every router logit (choice
+    and weights)."""
 
     kind: str
     ff: int
@@ -162,6 +175,7 @@ class MlpSpec:
     gated: bool = True
     shared_gate: bool = True
     table_rows: int = 0
+    router_bias: bool = False
 
 
 @dataclass
@@ -181,6 +195,8 @@ class LayerSpec:
     # joins the residual stream, and then scaled per channel (`layer_scale`)
     post_norm: bool = False
     layer_scale: bool = False
+    # False: the sublayers read the residual stream itself
+    pre_norm: bool = True
     # "rms" or "layer" (mean removed, weight and bias)
     norm: str = "rms"
     # taps of the causal per-channel convolution over time that every
@@ -849,6 +865,69 @@ ARCHITECTURES.update({
         "lusolix-8b", 4096, 128256, 32, heads=32, dim=128, rot_dim=64,
         vdim=128, kv_rank=512, q_rank=1536, window=2048, ff=14336,
         experts=8, top=2, expert_ff=3584, taps=4, positions=8192),
+})
+
+
+def _ralepel_stack(
+    name: str, width: int, vocab: int, n_layers: int, *, heads: int,
+    kv_heads: int, dim: int, window: int, lat_heads: int, lat_dim: int,
+    rot_dim: int, vdim: int, kv_rank: int, ff: int, experts: int, top: int,
+    expert_ff: int, shared_ff: int, rot_base: float = 500000.0,
+) -> ModelConfig:
+    """A Ralepel stack in the repeating order window, window, latent, window,
+    window, latent on the previous latent layer's cache; a dense feed-forward
+    in the first layer and routed experts with a gated shared expert in the
+    others; norms on the sublayers' outputs only."""
+    specs = []
+    for i in range(n_layers):
+        if i % 3 < 2:
+            mixer = MixerSpec(
+                kind="attention", heads=heads, kv_heads=kv_heads, dim=dim,
+                vdim=dim, scale=dim ** -0.5, window=window, sink=True,
+                learned_sink=True, bias=True, out_bias=True, rope=False,
+                key_values=True, unit_qk=True, distance_bias=True)
+        else:
+            mixer = MixerSpec(
+                kind="latent_attention", heads=lat_heads, kv_heads=1,
+                dim=lat_dim, vdim=vdim, kv_rank=kv_rank, rot_dim=rot_dim,
+                rot_dims=rot_dim, rot_base=rot_base, rot_layout="half",
+                scale=(lat_dim + rot_dim) ** -0.5, rope=True,
+                kv_from=i - 3 if i % 6 == 5 else None)
+        if i == 0:
+            mlp = MlpSpec(kind="dense", ff=ff, act="silu")
+        else:
+            mlp = MlpSpec(kind="moe", ff=expert_ff, act="silu",
+                          experts=experts, top=top, score="softmax",
+                          renormalize=True, router_bias=True,
+                          shared_ff=shared_ff)
+        specs.append(LayerSpec(mixer=mixer, mlp=mlp, parallel=False,
+                               post_norm=True, pre_norm=False))
+    return ModelConfig(
+        name=name, family="ralepel", hidden_size=width,
+        num_layers=n_layers, num_q_heads=heads, num_kv_heads=kv_heads,
+        head_dim=dim, intermediate_size=max(ff, expert_ff, shared_ff),
+        vocab_size=vocab, max_position=8192, layer_specs=specs,
+        bos_token_id=0, eos_token_id=-1)
+
+
+ARCHITECTURES.update({
+    # CPU-runnable test config
+    "tiny-ralepel": _ralepel_stack(
+        "tiny-ralepel", 80, 384, 6, heads=6, kv_heads=3, dim=16, window=24,
+        lat_heads=5, lat_dim=12, rot_dim=8, vdim=20, kv_rank=28, ff=160,
+        experts=5, top=2, expert_ff=32, shared_ff=48),
+    # llama-3.2-1b-sized stack (same width, depth, dense ff and vocab)
+    "ralepel-1b": _ralepel_stack(
+        "ralepel-1b", 2048, 128256, 16, heads=32, kv_heads=8, dim=64,
+        window=1024, lat_heads=32, lat_dim=64, rot_dim=32, vdim=64,
+        kv_rank=256, ff=8192, experts=8, top=2, expert_ff=2048,
+        shared_ff=2048),
+    # llama-3-8b-sized layers (width 4096, head dim 128, ff 14336)
+    "ralepel-8b": _ralepel_stack(
+        "ralepel-8b", 4096, 128256, 32, heads=32, kv_heads=8, dim=128,
+        window=2048, lat_heads=32, lat_dim=128, rot_dim=64, vdim=128,
+        kv_rank=512, ff=14336, experts=8, top=2, expert_ff=3584,
+        shared_ff=3584),
 })
 
 

@@ -187,6 +187,17 @@ class ModelRunner:
                     _, heads, d = desc
                     return torch.zeros((num_blocks, heads, bs, d), dtype=dt,
                                        device=self.device)
+                if kind == "keyval":
+                    # one paged tensor (raw keys that are the values) and
+                    # a fp32 factor per key
+                    _, heads, d = desc
+                    return (
+                        torch.zeros((num_blocks, heads, bs, d), dtype=dt,
+                                    device=self.device),
+                        torch.zeros((num_blocks, heads, bs),
+                                    dtype=torch.float32,
+                                    device=self.device),
+                    )
                 if kind == "state":
                     _, heads, d, dv = desc
                     return torch.zeros((slots, heads, d, dv),
@@ -202,7 +213,12 @@ class ModelRunner:
                     return tuple(alloc(d) for d in desc[1])
                 raise ValueError(f"unknown cache kind {kind!r}")
 
-            self.kv_caches = [alloc(d) for d in self.model.cache_shapes()]
+            self.kv_caches = []
+            for desc in self.model.cache_shapes():
+                # ("layer", j): the cache of an earlier layer
+                self.kv_caches.append(
+                    self.kv_caches[desc[1]] if desc[0] == "layer"
+                    else alloc(desc))
             return
         kh = self.model.kv_heads
         kv_dt = self.config.cache.kv_cache_dtype

@@ -213,6 +213,9 @@ class SparseMoE(nn.Module):
         self.correction = (
             nn.Parameter(torch.empty(E + spec.identity, dtype=torch.float32))
             if spec.correction else None)
+        self.router_bias = (
+            nn.Parameter(torch.empty(E + spec.identity, dtype=torch.float32))
+            if spec.router_bias else None)
         # without a gate branch the tensor holds the up rows only
         self.experts_gate_up = nn.Parameter(
             torch.empty(E, (2 if spec.gated else 1) * ff, width,
@@ -417,7 +420,8 @@ class SparseMoE(nn.Module):
         # one kernel: logits, scores, choice, weights, dense weight matrix
         weights, sel, wm = ops.moe_route(
             x, self.router, sp.top, sp.score, sp.renormalize,
-            self.correction, sp.route_scale, sp.renorm_eps)
+            self.correction, sp.route_scale, sp.renorm_eps,
+            self.router_bias)
         n_out = sp.experts + sp.identity
         small = dense if dense is not None else T <= self.GROUPED_MAX_ROWS
         if small and not self._grouped_fits(x):

@@ -48,7 +48,13 @@ class TalkAttention(nn.Module):
     behind the window stay visible through one mean key/value each, kept in
     a pooled cache that shares the pages of the key/value cache;
     `qk_norm_all`: query and key are normalised over their whole
-    projections."""
+    projections. `key_values` with `unit_qk`: the projected keys are the
+    values, and query and key heads are divided by their root mean square.
+    The cache then holds one row per position and KV head, the key as
+    projected, plus a fp32 number per row (one over its root mean square)
+    that multiplies the row's scores: half the bytes of a key/value cache,
+    and the norm is never rounded. `distance_bias`: linear penalty on the
+    distance of query and key, one slope per head."""
 
     kind = "attention"
 
@@ -68,8 +74,18 @@ class TalkAttention(nn.Module):
         if H % G:
             raise ValueError("heads must be a multiple of kv_heads")
         self.H, self.G, self.D, self.DV = H, G, D, DV
-        # fused rows: q | k | v (| output gate)
-        self.qkv_rows = H * D + G * D + G * DV
+        if spec.key_values != spec.unit_qk:
+            raise NotImplementedError(
+                "keys that are the values come with unit-rms queries and "
+                "keys, and the other way round")
+        if spec.key_values and (
+                DV != D or spec.rope or spec.qk_norm or spec.qk_norm_all
+                or spec.v_mix or spec.window_pool or spec.talking_heads):
+            raise NotImplementedError(
+                "keys that are the values: one width for both, no rotation, "
+                "learned norm, value blend, pooled blocks or head mix")
+        # fused rows: q | k | v (| output gate); no v where keys are values
+        self.qkv_rows = H * D + G * D + (0 if spec.key_values else G * DV)
         self.qkv = nn.Parameter(torch.empty(
             self.qkv_rows + (H * DV if spec.out_gate else 0), width,
             dtype=dtype))
@@ -104,6 +120,7 @@ class TalkAttention(nn.Module):
         self.vmix = (
             nn.Parameter(torch.empty((), dtype=torch.float32))
             if spec.v_mix else None)
+        self._slopes = None
 
     def in_params(self):
         return [self.qkv]
@@ -121,6 +138,17 @@ class TalkAttention(nn.Module):
                                 device, sp.rot_factor, sp.rot_scaling)
             self._cos_sin = cs
         return cs
+
+    def slopes(self, device) -> Optional[torch.Tensor]:
+        """fp32 [heads] distance slopes 2^(-8 (h + 1) / heads), or None."""
+        if not self.spec.distance_bias:
+            return None
+        sl = self._slopes
+        if sl is None or sl.device != device:
+            h = torch.arange(1, self.H + 1, dtype=torch.float64)
+            sl = self._slopes = torch.pow(
+                2.0, -8.0 * h / self.H).float().to(device)
+        return sl
 
     def project(self, o: torch.Tensor) -> torch.Tensor:
         if self.out_bias is not None:
@@ -141,6 +169,8 @@ class TalkAttention(nn.Module):
         return self.H * self.DV
 
     def cache_shape(self):
+        if self.spec.key_values:
+            return ("keyval", self.G, self.D)
         if self.spec.window_pool:
             return ("kvpool", self.G, self.D, self.DV,
                     self.spec.window_pool)
@@ -151,8 +181,11 @@ class TalkAttention(nn.Module):
                           shared: Optional[dict] = None) -> torch.Tensor:
         H, G, D, DV = self.H, self.G, self.D, self.DV
         sp = self.spec
-        pool = None
-        if sp.window_pool:
+        pool = key_scale = None
+        if sp.key_values:
+            k_cache, key_scale = cache
+            v_cache = k_cache
+        elif sp.window_pool:
             k_cache, v_cache, kp_cache, vp_cache = cache
             pool = (kp_cache, vp_cache, sp.window_pool)
         else:
@@ -160,7 +193,10 @@ class TalkAttention(nn.Module):
         q = proj[:, :H * D]
         k = proj[:, H * D:H * D + G * D]
         v = proj[:, H * D + G * D:self.qkv_rows]
-        if sp.qk_norm or sp.qk_norm_all or sp.v_mix or sp.rope:
+        if sp.key_values:
+            ops.keyval_prep(q, k, self.eps, k_cache, key_scale,
+                            meta.slot_mapping, H)
+        elif sp.qk_norm or sp.qk_norm_all or sp.v_mix or sp.rope:
             # the first value-mixing layer of a step publishes its values;
             # later ones blend theirs with them before caching
             v_first = shared.get("v_first") if sp.v_mix else None
@@ -198,7 +234,8 @@ class TalkAttention(nn.Module):
                     chunk=sp.chunk, window=sp.window, sink=sp.sink,
                     talk=self.talk, out=out[a:b], variant=variant,
                     keep_first=sp.keep_first, softcap=sp.softcap,
-                    sink_vals=self.sink_vals, pool=pool)
+                    sink_vals=self.sink_vals, pool=pool,
+                    key_scale=key_scale, slopes=self.slopes(proj.device))
         if sp.out_gate:
             ops.gated_act(proj[:, self.qkv_rows:], out, "sigmoid", out=out)
         return out
@@ -274,7 +311,9 @@ class LatentAttention(nn.Module):
     kv_rank + rot_dim numbers per token are cached. `window` limits the
     visible keys to the trailing ones; with `q_rank` the queries pass a
     normalised latent of their own; with `head_gate` every head's output is
-    multiplied by the sigmoid of one projected number.
+    multiplied by the sigmoid of one projected number. With `kv_from` the
+    layer has no latent: its cache is an earlier layer's, whose rows it reads
+    through up-projections of its own.
 
     Prompt portions that are not tiny against the keys they see take the
     unfolded form instead: the visible cached rows are gathered and expanded
@@ -301,8 +340,10 @@ class LatentAttention(nn.Module):
         # fused rows: q (per head [dim | rot_dim]) or its latent | latent |
         # rotary key (| head gates)
         self.q_rows = spec.q_rank or H * (D + R)
+        # rows of the latent and the rotary key part
+        self.kv_rows = L + R if spec.kv_from is None else 0
         self.in_proj = nn.Parameter(torch.empty(
-            self.q_rows + L + R + (H if spec.head_gate else 0), width,
+            self.q_rows + self.kv_rows + (H if spec.head_gate else 0), width,
             dtype=dtype))
         self.q_norm = self.uq = None
         if spec.q_rank:
@@ -310,7 +351,11 @@ class LatentAttention(nn.Module):
                 torch.empty(spec.q_rank, dtype=torch.float32))
             self.uq = nn.Parameter(
                 torch.empty(H * (D + R), spec.q_rank, dtype=dtype))
-        self.latent_norm = nn.Parameter(torch.empty(L, dtype=torch.float32))
+        self.latent_norm = (
+            nn.Parameter(torch.empty(L, dtype=torch.float32))
+            if spec.kv_from is None else None)
+        if spec.rot_layout not in ("interleaved", "half"):
+            raise ValueError(f"unknown rotary layout {spec.rot_layout!r}")
         self.uk = nn.Parameter(torch.empty(H, D, L, dtype=dtype))
         # transposed against the checkpoint's rows: both folded products
         # then read a contiguous right operand
@@ -377,13 +422,18 @@ class LatentAttention(nn.Module):
                 return None
         return plan
 
-    def _attend_expanded(self, q, plan, meta, cache, gate, out) -> None:
+    def _attend_expanded(self, q, plan, meta, cache, gate, out,
+                         shared: dict) -> None:
         """Attention of the portions' queries q [n, H*(dim+rot_dim)] over
         expanded keys and values, head gates included."""
         H, D, R, L, DV = self.H, self.D, self.R, self.L, self.DV
         sp, n, N = self.spec, q.shape[0], plan.total
-        rows = ops.latent_gather(cache, meta.block_tables, plan.segments, N,
-                                 plan.longest)
+        # layers on one cache (and with one window) gather its rows once
+        key = ("latent_rows", cache.data_ptr(), sp.window)
+        rows = shared.get(key)
+        if rows is None:
+            rows = shared[key] = ops.latent_gather(
+                cache, meta.block_tables, plan.segments, N, plan.longest)
         wk, wv = self.unfolded()
         k = F.linear(rows, wk)
         if ops.expanded_attention_fits(q, D + R, DV, sp.softcap):
@@ -408,6 +458,8 @@ class LatentAttention(nn.Module):
         return self.H * self.DV
 
     def cache_shape(self):
+        if self.spec.kv_from is not None:
+            return ("layer", self.spec.kv_from)
         return ("paged", 1, self.L + self.R)
 
     def cos_sin(self, device) -> torch.Tensor:
@@ -426,25 +478,28 @@ class LatentAttention(nn.Module):
         T = h.shape[0]
         proj = gemm_policy.linear(h, self.in_proj)
         q = proj[:, :self.q_rows]
-        dkv = proj[:, self.q_rows:self.q_rows + L + R]
+        kv_end = self.q_rows + self.kv_rows
+        dkv = proj[:, self.q_rows:kv_end] if self.kv_rows else None
         if self.q_rank:
             q = gemm_policy.linear(
                 ops.rms_norm_rows(q, self.q_norm, self.eps), self.uq)
         o = out if out is not None else torch.empty(
             (T, H * DV), dtype=h.dtype, device=h.device)
-        gate = proj[:, self.q_rows + L + R:] if sp.head_gate else None
+        gate = proj[:, kv_end:] if sp.head_gate else None
         cs, rd = self.cos_sin(h.device), sp.rot_dims or R
+        half = sp.rot_layout == "half"
         npt = min(getattr(meta, "num_prefill_tokens", T) or 0, T)
         plan = self._expansion(meta, npt, shared)
         n = npt if plan is not None else 0
         if n:
             qn = q[:n]
-            ops.latent_prep(None, qn, dkv[:n], self.latent_norm, self.eps,
-                            cs, meta.positions[:n], cache,
-                            meta.slot_mapping[:n], H, D, R, rd)
+            ops.latent_prep(None, qn, dkv[:n] if dkv is not None else None,
+                            self.latent_norm, self.eps, cs,
+                            meta.positions[:n], cache,
+                            meta.slot_mapping[:n], H, D, R, rd, half)
             self._attend_expanded(qn, plan, meta, cache,
                                   gate[:n] if gate is not None else None,
-                                  o[:n])
+                                  o[:n], shared)
         if n == T:
             return o
         # position-free query part into the latent space: [H, T, L]
@@ -452,8 +507,9 @@ class LatentAttention(nn.Module):
         q_lat = torch.bmm(q.view(m, H, D + R)[:, :, :D].transpose(0, 1),
                           self.uk)
         qf = ops.latent_prep(
-            q_lat, q, dkv[n:], self.latent_norm, self.eps, cs,
-            meta.positions[n:], cache, meta.slot_mapping[n:], H, D, R, rd)
+            q_lat, q, dkv[n:] if dkv is not None else None, self.latent_norm,
+            self.eps, cs, meta.positions[n:], cache, meta.slot_mapping[n:],
+            H, D, R, rd, half)
         o_lat = torch.empty((m, H * L), dtype=h.dtype, device=h.device)
         for a, b, variant in ((n, npt, 0), (npt, T, 3)):
             if b > a:

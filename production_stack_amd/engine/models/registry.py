@@ -61,6 +61,14 @@ def _lusolix_cls():
     return LusolixForCausalLM
 
 
+def _ralepel_cls():
+    from production_stack_amd.engine.models.ralepel import (
+        RalepelForCausalLM,
+    )
+
+    return RalepelForCausalLM
+
+
 MODEL_CLASSES: Dict[str, Callable] = {
     "llama": _llama_cls,
     "nanurax": _nanurax_cls,
@@ -68,6 +76,7 @@ MODEL_CLASSES: Dict[str, Callable] = {
     "bipulorn": _bipulorn_cls,
     "dogidra": _dogidra_cls,
     "lusolix": _lusolix_cls,
+    "ralepel": _ralepel_cls,
 }
 
 
@@ -102,16 +111,24 @@ def _lusolix_config(path: str) -> ModelConfig:
     return lusolix.config_from_dir(path)
 
 
+def _ralepel_config(path: str) -> ModelConfig:
+    from production_stack_amd.engine.models import ralepel
+
+    return ralepel.config_from_dir(path)
+
+
 CONFIG_READERS: Dict[str, Callable[[str], ModelConfig]] = {
     "Nanurax": _nanurax_config,
     "Derusun": _derusun_config,
     "Bipulorn": _bipulorn_config,
     "Dogidra": _dogidra_config,
     "Lusolix": _lusolix_config,
+    "Ralepel": _ralepel_config,
 }
 
 # families whose layers also run in float32 (the Llama path is bf16-only)
-FP32_FAMILIES = {"nanurax", "derusun", "bipulorn", "dogidra", "lusolix"}
+FP32_FAMILIES = {"nanurax", "derusun", "bipulorn", "dogidra", "lusolix",
+                 "ralepel"}
 
 
 def config_from_dir(path: str) -> ModelConfig:

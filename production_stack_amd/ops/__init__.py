@@ -623,7 +623,8 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
                    out: torch.Tensor = None, variant: int = 0,
                    splits: int = 0, keep_first: int = 0,
                    softcap: float = 0.0, sink_vals: torch.Tensor = None,
-                   vdim: int = 0, pool=None) -> torch.Tensor:
+                   vdim: int = 0, pool=None, key_scale: torch.Tensor = None,
+                   slopes: torch.Tensor = None) -> torch.Tensor:
     """Paged attention of a ragged batch. q [T, H*D] (row-strided view
     allowed); token_seq/token_pos int32 [T] give each token's block-table
     row and position; talk: optional fp32 [H, H] score mix; chunk/window:
@@ -635,7 +636,10 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     k_cache itself: keys that carry their values). pool = (kp_cache,
     vp_cache, P): with a window, every block of P positions that lies
     wholly before a query's window adds its pooled key and value (as
-    pool_append stores them) to the same softmax.
+    pool_append stores them) to the same softmax. key_scale fp32 [NB, G,
+    BS]: the scores of a key are multiplied by its number; slopes fp32 [H]:
+    slopes[h] * (query position - key position) is taken off the scaled
+    scores (neither comes with a head mix, a cap or pooled blocks).
     variant 0 picks the kernel for prompt portions (tiled thread-per-
     (head, query) where the shape fits), 3 for single tokens (split-key),
     both falling back to the plain one-workgroup-per-token kernel; 1 / 2 /
@@ -643,7 +647,9 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     and aligned chunks take the matrix-core kernel instead when the shape
     fits it (variants 0 and 3; 5 insists on it, 6 on its 128-row form);
     single tokens over rows that carry their values take a kernel of their
-    own first (variant 3; 7 insists on it).
+    own first (variant 3; 7 insists on it), and so do prompt portions and
+    single tokens over scaled keys that are their own values, whole rows
+    (variants 0 and 3; 8 and 9 insist on the portion / token form).
     Returns [T, H*DV]."""
     NB, G, BS, D = k_cache.shape
     VR = v_cache.shape[3]
@@ -660,6 +666,14 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     if sink_vals is not None:
         assert sink and sink_vals.dtype == torch.float32
         assert sink_vals.shape == (H,)
+    extra = key_scale is not None or slopes is not None
+    if extra:
+        assert talk is None and softcap == 0.0 and pool is None
+    if key_scale is not None:
+        assert key_scale.dtype == torch.float32
+        assert key_scale.shape == (NB, G, BS)
+    if slopes is not None:
+        assert slopes.dtype == torch.float32 and slopes.shape == (H,)
     kp = vp = None
     P = PR = 0
     if pool is not None and window > 0:
@@ -677,10 +691,12 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
         o = reference.talk_attention(
             q.reshape(T, H, D), k_cache, v_cache, block_tables, token_seq,
             token_pos, scale, chunk, window, sink, talk, keep_first,
-            softcap, sink_vals, DV, pool)
+            softcap, sink_vals, DV, pool, key_scale, slopes)
         out.copy_(o.reshape(T, H * DV))
         return out
     assert q.dtype == k_cache.dtype == v_cache.dtype
+    for t in (key_scale, slopes):
+        assert t is None or t.is_contiguous()
     assert k_cache.is_contiguous() and v_cache.is_contiguous()
     assert block_tables.is_contiguous()
     if talk is not None:
@@ -692,7 +708,7 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     # workgroups whose partial softmax records are merged afterwards
     scratch = None
     if (variant in (3, 7) and q.dtype == torch.bfloat16 and G == 1
-            and v_cache.data_ptr() == k_cache.data_ptr() and talk is None
+            and not extra and v_cache.data_ptr() == k_cache.data_ptr() and talk is None
             and chunk == 0 and keep_first == 0 and softcap == 0.0):
         shares = splits if splits > 0 else max(
             1, min(16 if T <= 4 else 8, 256 // (T * ((H + 31) // 32))))
@@ -720,7 +736,7 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     # bf16 without head mix / aligned chunks: the matrix-core kernel, where
     # the shape fits it (variant 5 insists on it)
     if (variant in (0, 3, 5, 6) and q.dtype == torch.bfloat16
-            and talk is None and chunk == 0):
+            and talk is None and chunk == 0 and not extra):
         # 0: prompt portions, 1: single tokens, 2: 128-row workgroups
         mode = (2 if variant == 6 else
                 int(variant == 3 or (variant == 5 and splits > 0)))
@@ -744,7 +760,7 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
         _f(scale), int(chunk), int(window), int(bool(sink)),
         _mx_dtype(q.dtype), int(variant), int(splits), _p(scratch),
         int(keep_first), _f(softcap), _p(sink_vals), int(VR), _p(kp),
-        _p(vp), int(P), _stream())
+        _p(vp), int(P), _p(key_scale), _p(slopes), _stream())
     if rc != 0:
         raise RuntimeError(
             f"talk_attention: heads x dim {H}x{D}/{DV} exceeds the kernel's "
@@ -803,6 +819,31 @@ def attn_prep(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
         _p(cos_sin), int(cos_sin.shape[0]) if cos_sin is not None else 0,
         int(rot_dims) if cos_sin is not None else 0, _p(positions),
         int(bool(norm_all)), int(bool(half)), _mx_dtype(q.dtype), _stream())
+
+
+def keyval_prep(q: torch.Tensor, k: torch.Tensor, eps: float,
+                cache: torch.Tensor, key_scale: torch.Tensor,
+                slot_mapping: torch.Tensor, heads: int) -> None:
+    """Inputs of attention whose keys are their own values: every query head
+    of q [T, H*D] is divided by its root mean square in place, the key rows
+    k [T, G*D] go to the paged cache [NB, G, BS, D] as they are, and
+    key_scale fp32 [NB, G, BS] receives one over their root mean square. q
+    and k are row-strided views."""
+    NB, G, BS, D = cache.shape
+    T, H = q.shape[0], heads
+    assert q.shape == (T, H * D) and k.shape == (T, G * D)
+    assert key_scale.dtype == torch.float32
+    assert key_scale.shape == (NB, G, BS)
+    assert slot_mapping.dtype == torch.long and slot_mapping.shape == (T,)
+    if not q.is_cuda:
+        reference.keyval_prep(q, k, eps, cache, key_scale, slot_mapping, H)
+        return
+    assert q.dtype == k.dtype == cache.dtype
+    assert cache.is_contiguous() and key_scale.is_contiguous()
+    _mx().mx_keyval_prep(
+        _p(q), _rows(q, "q"), _p(k), _rows(k, "k"), _f(eps), _p(cache),
+        _p(key_scale), _p(slot_mapping), T, H, G, D, BS, _mx_dtype(q.dtype),
+        _stream())
 
 
 def rope_table(max_pos: int, dims: int, base: float,
@@ -1133,16 +1174,20 @@ def latent_prep(q_lat: torch.Tensor, q: torch.Tensor, dkv: torch.Tensor,
                 norm_w: torch.Tensor, eps: float, cos_sin: torch.Tensor,
                 positions: torch.Tensor, cache: torch.Tensor,
                 slot_mapping: torch.Tensor, heads: int, dim: int,
-                rot_dim: int, rot_dims: int) -> torch.Tensor:
+                rot_dim: int, rot_dims: int,
+                half: bool = False) -> torch.Tensor:
     """Inputs of latent attention (see reference.latent_prep): normalises
     the latent, turns the shared key part and the queries' rotated parts
     by their positions, appends [latent | key part] to the paged cache
     [NB, 1, BS, L+rot_dim] and returns the queries [T, H*(L+rot_dim)].
     q_lat None: the queries stay [position-free | rotated] per head; their
-    rotated parts turn in place in q, which is returned."""
+    rotated parts turn in place in q, which is returned. dkv None: nothing
+    is appended (the cache is another layer's). half: the rotary pairs are
+    (i, i + rot_dims/2) instead of neighbours."""
     H = heads
     T = q.shape[0]
-    L = dkv.shape[1] - rot_dim
+    L = cache.shape[3] - rot_dim
+    assert dkv is None or dkv.shape == (T, L + rot_dim)
     assert q.shape == (T, H * (dim + rot_dim))
     if q_lat is not None:
         assert q_lat.shape == (H, T, L) and q_lat.is_contiguous()
@@ -1156,9 +1201,11 @@ def latent_prep(q_lat: torch.Tensor, q: torch.Tensor, dkv: torch.Tensor,
     if not q.is_cuda:
         return reference.latent_prep(
             q_lat, q, dkv, norm_w, eps, cos_sin, positions, cache,
-            slot_mapping, H, dim, rot_dim, rot_dims, q.dtype)
-    assert q.dtype == dkv.dtype == cache.dtype
-    assert norm_w.dtype == torch.float32 and norm_w.numel() == L
+            slot_mapping, H, dim, rot_dim, rot_dims, q.dtype, half)
+    assert q.dtype == cache.dtype
+    if dkv is not None:
+        assert dkv.dtype == q.dtype
+        assert norm_w.dtype == torch.float32 and norm_w.numel() == L
     assert cache.is_contiguous() and cos_sin.is_contiguous()
     out = q
     if q_lat is not None:
@@ -1166,10 +1213,11 @@ def latent_prep(q_lat: torch.Tensor, q: torch.Tensor, dkv: torch.Tensor,
                           device=q.device)
     _mx().mx_latent_prep(
         _p(out), _p(q_lat), _p(q), _rows(q, "q"), _p(dkv),
-        _rows(dkv, "dkv"), _p(norm_w), _f(eps), _p(cos_sin),
+        _rows(dkv, "dkv") if dkv is not None else 0,
+        _p(norm_w if dkv is not None else None), _f(eps), _p(cos_sin),
         int(cos_sin.shape[0]), int(rot_dims), _p(positions), _p(cache),
         _p(slot_mapping), T, H, dim, rot_dim, L, cache.shape[2],
-        _mx_dtype(q.dtype), _stream())
+        int(bool(half)), _mx_dtype(q.dtype), _stream())
     return out
 
 
@@ -1317,17 +1365,20 @@ def norm_sum32(inputs, weights, scale: float, eps: float) -> torch.Tensor:
 
 
 def post_norm_add_norm32(x32: torch.Tensor, delta: torch.Tensor,
-                         w_post: torch.Tensor, w_next: torch.Tensor,
+                         w_post: torch.Tensor, w_next,
                          eps: float, out_dtype: torch.dtype) -> torch.Tensor:
     """Sublayer boundary of a stack that normalises a sublayer's output
     before it joins the residual stream: x32 += rmsnorm(delta) * w_post
     (fp32 [T, W], in place; delta [T, W] fp32 or the serving dtype,
     row-strided view allowed), returns rmsnorm(x32) * w_next in out_dtype:
-    the next sublayer's input. Weights fp32 [W]."""
+    the next sublayer's input. Weights fp32 [W]; w_next None: the input is
+    x32 itself, rounded."""
     T, W = x32.shape
     assert x32.dtype == torch.float32 and x32.is_contiguous()
     assert delta.shape == (T, W)
     for w in (w_post, w_next):
+        if w is None:
+            continue
         assert w.dtype == torch.float32 and w.numel() == W
     if not x32.is_cuda:
         return reference.post_norm_add_norm32(x32, delta, w_post, w_next,
@@ -1424,10 +1475,10 @@ def linear_scan(mode: str, q, k, v, dec, gate, state, seq_rows, heads: int,
 def moe_route(x: torch.Tensor, router_w: torch.Tensor, top: int,
               score: str = "softmax", renormalize: bool = True,
               correction: torch.Tensor = None, scale: float = 1.0,
-              renorm_eps: float = 0.0):
+              renorm_eps: float = 0.0, bias: torch.Tensor = None):
     """Router of a routed feed-forward in one kernel (see
     reference.moe_route): fp32 logits of x [T, W] against router_w
-    [n_out, W] (both of the serving dtype), softmax or sigmoid scores, the
+    [n_out, W] (both of the serving dtype) plus bias (fp32 [n_out]), softmax or sigmoid scores, the
     `top` best by score + correction (fp32 [n_out]), weights
     = chosen scores / (sum + renorm_eps) when renormalize, times scale.
     Returns (weights fp32 [T, top], indices int64 [T, top], dense fp32
@@ -1437,19 +1488,20 @@ def moe_route(x: torch.Tensor, router_w: torch.Tensor, top: int,
     n_out = router_w.shape[0]
     assert router_w.shape == (n_out, W) and router_w.dtype == x.dtype
     assert score in ("softmax", "sigmoid") and 1 <= top <= n_out
-    if correction is not None:
-        assert correction.dtype == torch.float32
-        assert correction.shape == (n_out,)
+    for v in (correction, bias):
+        assert v is None or (v.dtype == torch.float32
+                             and v.shape == (n_out,))
     if not x.is_cuda:
         return reference.moe_route(x, router_w, top, score, renormalize,
-                                   correction, scale, renorm_eps)
+                                   correction, scale, renorm_eps, bias)
     assert router_w.is_contiguous()
     sel = torch.empty((T, top), dtype=torch.long, device=x.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=x.device)
     dense = torch.empty((T, n_out), dtype=torch.float32, device=x.device)
     rc = _mx().mx_moe_route(
         _p(sel), _p(wts), _p(dense), _p(x), _rows(x, "x"), _p(router_w),
-        _p(correction), T, W, n_out, int(top), int(score == "sigmoid"),
+        _p(correction), _p(bias), T, W, n_out, int(top),
+        int(score == "sigmoid"),
         int(bool(renormalize)), _f(renorm_eps), _f(scale),
         _mx_dtype(x.dtype), _stream())
     if rc != 0:

@@ -306,7 +306,8 @@ def kv_append(k, v, k_cache, v_cache, slot_mapping) -> None:
 def talk_attention(q, k_cache, v_cache, block_tables, token_seq, token_pos,
                    scale: float, chunk: int, window: int, sink: bool,
                    talk, keep_first: int = 0, softcap: float = 0.0,
-                   sink_vals=None, vdim: int = 0, pool=None):
+                   sink_vals=None, vdim: int = 0, pool=None, key_scale=None,
+                   slopes=None):
     """Paged attention with optional head-mixed scores, aligned-chunk or
     trailing-window visibility (the first keep_first keys stay visible
     behind the window), capped scores and a denominator sink (score 0, or
@@ -315,7 +316,9 @@ def talk_attention(q, k_cache, v_cache, block_tables, token_seq, token_pos,
     [T, H, DV] in q's dtype; all score math in fp32. pool = (kp_cache,
     vp_cache, P): with a window, every block of P positions whose last
     position is at or before pos - window adds its pooled key/value (see
-    pool_append) to the same softmax."""
+    pool_append) to the same softmax. key_scale [NB, G, BS]: a number per
+    key that multiplies its scores; slopes [H]: slopes[h] * (pos - key
+    position) is taken off the scaled scores."""
     T, H, D = q.shape
     G, bs = v_cache.shape[1], v_cache.shape[2]
     DV = vdim or v_cache.shape[3]
@@ -348,6 +351,10 @@ def talk_attention(q, k_cache, v_cache, block_tables, token_seq, token_pos,
         kk = kk.repeat_interleave(rep, dim=1)      # [n, H, D]
         vv = vv.repeat_interleave(rep, dim=1)
         s = torch.einsum("hd,nhd->hn", q[t].float(), kk) * scale
+        if key_scale is not None:
+            s = s * key_scale[blk, :, off].repeat_interleave(rep, dim=1).t()
+        if slopes is not None:
+            s = s - slopes.view(H, 1) * (pos - idx).float()
         if tk is not None:
             s = tk @ s
         if softcap > 0:
@@ -403,6 +410,21 @@ def attn_prep(q, k, v, q_w, k_w, eps: float, vmix, v_first, k_cache,
         vf = (1.0 - lam) * vf + lam * v_first.float()
         v.copy_(vf.to(v.dtype))
     kv_append(kf, vf.view(T, G, DV), k_cache, v_cache, slot_mapping)
+
+
+def keyval_prep(q, k, eps: float, cache, key_scale, slot_mapping,
+                heads: int) -> None:
+    """q [T, H*D] over its root mean square per head, in place; k [T, G*D]
+    appended to cache [NB, G, BS, D] as it is, one over its root mean square
+    per head to key_scale fp32 [NB, G, BS]."""
+    T = q.shape[0]
+    G, bs, D = cache.shape[1], cache.shape[2], cache.shape[3]
+    q.copy_(_unit_heads(q.float().view(T, heads, D), eps, False)
+            .reshape(T, heads * D).to(q.dtype))
+    kf = k.float().view(T, G, D)
+    blk, off = (slot_mapping // bs).long(), (slot_mapping % bs).long()
+    cache[blk, :, off] = kf.to(cache.dtype)
+    key_scale[blk, :, off] = torch.rsqrt(kf.pow(2).mean(-1) + eps)
 
 
 def _unit_heads(x, eps: float, whole: bool):
@@ -587,7 +609,7 @@ def mingru_scan(z, u, g, zb, ub, state, seq_rows, out_dtype):
 
 def latent_prep(q_lat, q, dkv, norm_w, eps: float, cos_sin, positions,
                 cache, slot_mapping, heads: int, dim: int, rot_dim: int,
-                rot_dims: int, out_dtype):
+                rot_dims: int, out_dtype, half: bool = False):
     """Inputs of latent attention for one step. q_lat [H, T, L]: the
     position-free query parts already mapped into the latent space; q
     [T, H*(dim+rot_dim)]: its rotated parts are taken and turned; dkv
@@ -595,20 +617,22 @@ def latent_prep(q_lat, q, dkv, norm_w, eps: float, cos_sin, positions,
     the latent, the rest is the shared rotated key part. The cache
     [NB, 1, BS, L+rot_dim] receives [latent | turned key part]; returns
     the queries [T, H*(L+rot_dim)] = per head [q_lat | turned part]; q_lat
-    None: q itself, its rotated parts turned in place."""
+    None: q itself, its rotated parts turned in place. dkv None: the cache
+    stays as it is. half: pairs (i, i + rot_dims/2)."""
     H = heads
     T = q.shape[0]
-    L = dkv.shape[1] - rot_dim
+    L = cache.shape[3] - rot_dim
     cs = cos_sin[positions.long()]                        # [T, dims/2, 2]
-    c = dkv[:, :L].float()
-    c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * norm_w
-    kr = _rotate(dkv[:, L:].float(), cs, rot_dims)
-    row = torch.cat([c, kr], dim=-1)
-    bs = cache.shape[2]
-    cache[(slot_mapping // bs).long(), 0, (slot_mapping % bs).long()] = \
-        row.to(cache.dtype)
+    if dkv is not None:
+        c = dkv[:, :L].float()
+        c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * norm_w
+        kr = _rotate(dkv[:, L:].float(), cs, rot_dims, half)
+        row = torch.cat([c, kr], dim=-1)
+        bs = cache.shape[2]
+        cache[(slot_mapping // bs).long(), 0, (slot_mapping % bs).long()] = \
+            row.to(cache.dtype)
     qr = q.float().view(T, H, dim + rot_dim)[..., dim:]
-    qr = _rotate(qr, cs[:, None], rot_dims)
+    qr = _rotate(qr, cs[:, None], rot_dims, half)
     if q_lat is None:
         q.view(T, H, dim + rot_dim)[..., dim:] = qr.to(q.dtype)
         return q
@@ -772,9 +796,12 @@ def norm_sum32(inputs, weights, scale: float, eps: float):
 
 def post_norm_add_norm32(x32, delta, w_post, w_next, eps: float, out_dtype):
     """x32 += rmsnorm(delta) * w_post (fp32, in place); returns
-    rmsnorm(x32) * w_next in out_dtype."""
+    rmsnorm(x32) * w_next in out_dtype (w_next None: x32 itself)."""
     d = delta.float()
     x32.add_(d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w_post)
+    if w_next is None:
+        # a copy: the stream moves on while the input is still read
+        return x32.to(out_dtype, copy=True)
     return (x32 * torch.rsqrt(x32.pow(2).mean(-1, keepdim=True) + eps)
             * w_next).to(out_dtype)
 
@@ -862,17 +889,17 @@ def linear_scan(mode: str, q, k, v, dec, wr, gate, p0, p1, p2, normw, state,
 
 
 def moe_route(x, router_w, top: int, score: str, renormalize: bool,
-              correction, scale: float, renorm_eps: float):
-    """Router of a routed feed-forward: fp32 logits, softmax | sigmoid
-    scores, the `top` outputs with the largest score + correction (sigmoid
-    scores without a correction are ranked by their logits), weights =
+              correction, scale: float, renorm_eps: float, bias=None):
+    """Router of a routed feed-forward: fp32 logits (+ bias), softmax | sigmoid
+    scores, the `top` outputs with the largest score + correction (scores
+    without a correction are ranked by their logits), weights =
     chosen scores, divided by
     (their sum + renorm_eps) when renormalize, times scale. Returns
     (weights [T, top], indices [T, top], dense [T, n_out])."""
-    logits = torch.nn.functional.linear(x.float(), router_w.float())
+    logits = torch.nn.functional.linear(x.float(), router_w.float(), bias)
     if score == "softmax":
         probs = torch.softmax(logits, dim=-1)
-        pick = probs + correction if correction is not None else probs
+        pick = probs + correction if correction is not None else logits
     else:
         probs = torch.sigmoid(logits)
         pick = probs + correction if correction is not None else logits
