@@ -335,6 +335,16 @@ __global__ __launch_bounds__(256) void latent_decode_combine_kernel(
   }
 }
 
+// Merge pass over partial records as above, at most 16 shares.
+extern "C" void mx_latent_combine(void* out, int ldout, const void* part,
+                                  int T_, int H, int DV, int KS,
+                                  void* stream) {
+  hipLaunchKernelGGL(latent_decode_combine_kernel, dim3(T_, H),
+                     dim3(DV <= 64 ? 64 : (DV <= 128 ? 128 : 256)), 0,
+                     (hipStream_t)stream, (unsigned short*)out, ldout,
+                     (const float*)part, H, DV, KS);
+}
+
 // Returns 0 when launched, 1 when the shape is outside this kernel: rows of
 // whole 16-byte vectors, up to 320 entries with at most 256 value columns or
 // up to 576 with at most 512.
@@ -367,10 +377,6 @@ extern "C" int mx_latent_decode(
   else
     LD_GO(18, 2);
 #undef LD_GO
-  if (KS > 1)
-    hipLaunchKernelGGL(latent_decode_combine_kernel, dim3(T_, H),
-                       dim3(DV <= 64 ? 64 : (DV <= 128 ? 128 : 256)), 0,
-                       (hipStream_t)stream, (U*)out, ldout,
-                       (const float*)scratch, H, DV, KS);
+  if (KS > 1) mx_latent_combine(out, ldout, scratch, T_, H, DV, KS, stream);
   return 0;
 }

@@ -725,6 +725,32 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     if variant == 7:
         raise RuntimeError(
             "talk_attention: shape or dtype outside the latent-row kernel")
+    # scaled keys that are their own values
+    if (variant in (0, 3, 8, 9) and extra and q.dtype == torch.bfloat16
+            and v_cache.data_ptr() == k_cache.data_ptr() and DV == D
+            and chunk == 0 and keep_first == 0):
+        token = variant in (3, 9)
+        shares = 1
+        if token:
+            # enough workgroups to fill the chip, a share being at least one
+            # tile of rows per wave
+            groups = T * G * ((H // G + 15) // 16)
+            shares = splits if splits > 0 else max(
+                1, min(16, 1024 // groups,
+                       (window + 127) // 128 if window > 0 else 16))
+        part = (torch.empty((T, shares, H, D + 4), dtype=torch.float32,
+                            device=q.device) if shares > 1 else None)
+        rc = _mx().mx_keyval_attention(
+            _p(out), _rows(out, "out"), _p(q), _rows(q, "q"), _p(k_cache),
+            _p(key_scale), _p(block_tables), block_tables.shape[1],
+            _p(token_seq), _p(token_pos), T, H, G, D, BS, _f(scale),
+            int(window), int(bool(sink)), _p(sink_vals), _p(slopes),
+            int(token), int(shares), _p(part), _stream())
+        if rc == 0:
+            return out
+    if variant in (8, 9):
+        raise RuntimeError(
+            "talk_attention: shape or dtype outside the key-value kernels")
     if variant not in (3, 4, 5, 6):
         splits = 1
     elif splits <= 0:

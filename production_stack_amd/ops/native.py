@@ -10,8 +10,8 @@ shape checks live in the Python wrappers
 
 Groups (one shared library each):
   core    resid32, norm_conv, mixer_prep, talk_attention, mfma_attention,
-          expand_attention, latent_decode, moe_route, moe_group,
-          mingru_scan                       -> _mixops.so
+          expand_attention, latent_decode, keyval_attention, moe_route,
+          moe_group, mingru_scan            -> _mixops.so
   delta   delta_rule                        -> _mixops_delta.so
   gdelta  gated_delta                       -> _mixops_gdelta.so
   scan    linear_scan                       -> _mixops_scan.so
@@ -48,6 +48,7 @@ GROUPS = {
         ("mfma_attention.hip", []),
         ("expand_attention.hip", []),
         ("latent_decode.hip", []),
+        ("keyval_attention.hip", []),
         ("moe_route.hip", []),
         ("moe_group.hip", []),
         ("mingru_scan.hip", []),
@@ -85,7 +86,7 @@ INT_RESULT = {
     "mx_short_conv_silu", "mx_mfma_attention", "mx_linear_scan",
     "mx_linear_scan_splits", "mx_norm_conv32", "mx_moe_route",
     "mx_add_layer_norm32", "mx_expert_plan", "mx_expand_attention",
-    "mx_latent_decode",
+    "mx_latent_decode", "mx_keyval_attention",
 }
 
 # entry points that return a 64-bit count
