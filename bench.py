@@ -115,7 +115,8 @@ class User:
 # first two; for Bipulorn the other hybrid with routed feed-forwards, whose
 # expert widths are the same; for Dogidra Bipulorn, whose pair layers also
 # put a windowed attention beside a recurrence ahead of a routed
-# feed-forward with a shared expert)
+# feed-forward with a shared expert; for Ralepel Lusolix, the other family of
+# latent attention and routed experts)
 COMPARE_PAIRS = {
     "nanurax": [("nanurax-1b", "llama-3.2-1b"), ("nanurax-8b", "llama-3-8b")],
     "derusun": [("derusun-1b", "llama-3.2-1b"), ("derusun-8b", "llama-3-8b")],
@@ -124,6 +125,7 @@ COMPARE_PAIRS = {
     "dogidra": [("dogidra-1b", "bipulorn-1b"),
                 ("dogidra-8b", "bipulorn-8b")],
     "lusolix": [("lusolix-1b", "dogidra-1b"), ("lusolix-8b", "dogidra-8b")],
+    "ralepel": [("ralepel-1b", "lusolix-1b"), ("ralepel-8b", "lusolix-8b")],
 }
 
 
