@@ -21,6 +21,13 @@
 //                   final merge of the four waves. v_mfma_f32_16x16x32_bf16
 //                   with up to 16 query heads as the narrow side.
 //
+// Tiles are walked from the nearest to the farthest: with a distance penalty the
+// running maximum then settles in the first tile or two. Where the caller knows
+// a bound B of |scale f_j q_i . r_j| (unit-rms queries and keys: scale D), keys
+// so far away that B - slope_h distance lies 40 powers of two below -B, the
+// least score of the query's own key, are not visited at all: their weights are
+// below 2^-40 of the largest one, far less than the rounding of the sum.
+//
 // In both, the rows of a score tile are read from LDS in an order that leaves
 // every lane with runs of 8 consecutive keys of one (token, head): the softmax
 // is lane-local plus exchanges between the lanes of one head, and the weights
@@ -60,6 +67,7 @@ struct KvArgs {
   int window, sink;
   const float* sink_vals;       // per head (nullptr: score 0)
   const float* slopes;          // per head (nullptr: no distance term)
+  float bound2;                 // bound of the scores times log2(e), < 0: none
   int KS;                       // shares (token kernel)
   float* part;
   int hpb, hblocks;             // heads per workgroup, head blocks per KV head
@@ -79,6 +87,49 @@ PS_DEV void kv_split(float p0, float p1, unsigned int* a, unsigned int* b,
   *a = __builtin_amdgcn_perm(x1, x0, 0x07060302u);
   *b = __builtin_amdgcn_perm(y1, y0, 0x07060302u);
   *c = __builtin_amdgcn_perm(z1, z0, 0x07060302u);
+}
+
+// Distance from which on no head of h0 .. h0 + n - 1 sees anything that counts
+// (see above); a large number where there is no such distance.
+PS_DEV int kv_reach(const KvArgs& a, int h0, int n) {
+  const int far = 1 << 30;
+  if (a.slopes == nullptr || a.bound2 < 0.f) return far;
+  float sl = a.slopes[h0];
+  for (int h = 1; h < n; ++h) sl = fminf(sl, a.slopes[h0 + h]);
+  if (!(sl > 0.f)) return far;
+  const float d = (2.0f * a.bound2 + 40.0f) / (sl * KV_LOG2E);
+  return d < 1.0e9f ? (int)d + 2 : far;
+}
+
+// One online-softmax step of a lane's N scores v (relative to the running
+// maximum m, or absolute while m is KV_LOW): weights into v, their sum into l,
+// the new maximum into m; returns the factor for what was accumulated before.
+// mx: the largest v over all lanes of the row. The factor is 1 for every lane
+// (and *moved false) when no maximum of the wave moves.
+template <int N>
+PS_DEV float kv_softmax(float* v, float mx, float* m, float* l, bool* moved) {
+  const bool fresh = *m == KV_LOW;
+  *moved = __any(mx > 0.f || (fresh && mx > -INFINITY));
+  float alpha = 1.f;
+  if (*moved) {
+    const float d = fresh ? (mx > -INFINITY ? mx : 0.f) : fmaxf(mx, 0.f);
+    if (!fresh) {
+      alpha = __builtin_amdgcn_exp2f(-d);
+      *m += d;
+    } else if (mx > -INFINITY) {
+      *m = d;
+    }
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] -= d;
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < N; ++i) {
+    v[i] = __builtin_amdgcn_exp2f(v[i]);
+    s += v[i];
+  }
+  *l = *l * alpha + s;
+  return alpha;
 }
 
 // ---------------------------------------------------------------------------
@@ -101,17 +152,11 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
   const int TPT = 128 / HPB;
   const int NT = (a.T + TPT - 1) / TPT;
 
-  // the tiles of one KV head on one XCD (workgroups go round the 8 of them)
-  int gh, tile;
+  // heavy workgroups first: later tiles, and the heads with the flattest
+  // slopes (the last ones of the usual geometric series)
   const int GH = a.G * a.hblocks;
-  if (GH % 8 == 0) {
-    const int k8 = blockIdx.x >> 3;
-    gh = (blockIdx.x & 7) + 8 * (k8 / NT);
-    tile = k8 % NT;
-  } else {
-    gh = blockIdx.x / NT;
-    tile = blockIdx.x % NT;
-  }
+  const int gh = GH - 1 - blockIdx.x / NT;
+  const int tile = NT - 1 - blockIdx.x % NT;
   const int g = gh / a.hblocks, hb = gh % a.hblocks;
   const int tok0 = tile * TPT, ntok = min(TPT, a.T - tok0);
   for (int c = tid; c < ntok; c += 256) {
@@ -129,6 +174,9 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
   const int my_pos = s_pos[min(my_i, ntok - 1)];
   const float sl2 =
       a.slopes != nullptr ? a.slopes[head] * KV_LOG2E : 0.f;
+  const int reach =
+      kv_reach(a, g * rep + hb * HPB, min(HPB, rep - hb * HPB));
+  const int span = a.window > 0 ? min(a.window, reach) : reach;
   // queries: B operand, lane (row, hi) holds entries 16 s + 8 hi + i
   kv_bf16x8 qr[DK];
   {
@@ -172,7 +220,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
     const bool mine = valid && my_i >= rs && my_i < re;
     const bool all_mine = __all(mine);
     const int* table = a.block_tables + (size_t)s_seq[rs] * a.max_blocks;
-    const int kmin = a.window > 0 ? max(0, s_pos[rs] - a.window + 1) : 0;
+    const int kmin = max(0, s_pos[rs] - span + 1);
     const int kmax = s_pos[re - 1];
     const int nt = (kmax - kmin) / KV_KT + 1;
     // rows of other runs see nothing of this one
@@ -190,7 +238,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
     auto find = [&](int n, int buf) {
       if (tid < KV_KT) {
         // rows past the last key repeat it; they are masked
-        const int j = min(kmin + n * KV_KT + tid, kmax);
+        const int j = min(kmin + (nt - 1 - n) * KV_KT + tid, kmax);
         s_row[buf][tid] = (table[j / a.BS] * a.G + g) * a.BS + (j % a.BS);
       }
     };
@@ -223,7 +271,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
       if (n + 2 < nt) find(n + 2, n & 1);
       __syncthreads();
       if (n + 1 < nt) fetch((n + 1) & 1);
-      const int j0 = kmin + n * KV_KT;
+      const int j0 = kmin + (nt - 1 - n) * KV_KT;
       if (!live || j0 > w_last || j0 + KV_KT - 1 < w_lo) continue;
 
       kv_f32x16 st[2];
@@ -240,7 +288,9 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
                                                         0, 0);
       }
       // st[h][8 s + i] belongs to key j0 + 32 h + 16 s + 8 hi + i
-      const float base = sl2 * (float)(j0 + 8 * hi - pos);
+      const float base =
+          sl2 * (float)(j0 + 8 * hi - pos) - (m == KV_LOW ? 0.f : m);
+      float w[32];
 #pragma unroll
       for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -251,7 +301,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
           const float f[8] = {f0.x, f0.y, f0.z, f0.w, f1.x, f1.y, f1.z, f1.w};
 #pragma unroll
           for (int i = 0; i < 8; ++i)
-            st[h][8 * s + i] =
+            w[16 * h + 8 * s + i] =
                 fmaf(st[h][8 * s + i], f[i],
                      fmaf(sl2, (float)(32 * h + 16 * s + i), base));
         }
@@ -261,27 +311,16 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int j = j0 + 32 * h + 16 * (r >> 3) + 8 * hi + (r & 7);
-            if (j > pos || j < lo) st[h][r] = -INFINITY;
+            if (j > pos || j < lo) w[16 * h + r] = -INFINITY;
           }
       }
-      float mx = st[0][0];
+      float mx = w[0];
 #pragma unroll
-      for (int r = 0; r < 16; ++r) mx = fmaxf(mx, fmaxf(st[0][r], st[1][r]));
+      for (int i = 1; i < 32; ++i) mx = fmaxf(mx, w[i]);
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mnew = fmaxf(m, mx);
-      const float alpha = __builtin_amdgcn_exp2f(m - mnew);
-      float ps = 0.f;
-#pragma unroll
-      for (int h = 0; h < 2; ++h)
-#pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          const float p = __builtin_amdgcn_exp2f(st[h][r] - mnew);
-          st[h][r] = p;
-          ps += p;
-        }
-      l = l * alpha + ps;
-      m = mnew;
-      if (__any(alpha != 1.f)) {
+      bool moved;
+      const float alpha = kv_softmax<32>(w, mx, &m, &l, &moved);
+      if (moved) {
 #pragma unroll
         for (int c = 0; c < CB; ++c)
 #pragma unroll
@@ -292,9 +331,8 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
         KvPack b0, b1, b2;
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          kv_split(st[s >> 1][8 * (s & 1) + 2 * i],
-                   st[s >> 1][8 * (s & 1) + 2 * i + 1], &b0.w[i], &b1.w[i],
-                   &b2.w[i]);
+          kv_split(w[8 * s + 2 * i], w[8 * s + 2 * i + 1], &b0.w[i],
+                   &b1.w[i], &b2.w[i]);
 #pragma unroll
         for (int c = 0; c < CB; ++c) {
           KvPack v;
@@ -367,13 +405,16 @@ __global__ __launch_bounds__(256, DK < 4 ? 4 : DK == 4 ? 3 : 1) void keyval_toke
   __shared__ float s_m[4][16], s_l[4][16];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int t = blockIdx.x, ks = blockIdx.z;
-  const int g = blockIdx.y / a.hblocks, hb = blockIdx.y % a.hblocks;
+  const int gh = gridDim.y - 1 - blockIdx.y;  // flattest slopes first
+  const int g = gh / a.hblocks, hb = gh % a.hblocks;
   const int D = a.D, rep = a.H / a.G;
   const int nh = min(16, rep - hb * 16);      // heads of this workgroup
   const int h0 = g * rep + hb * 16;
   const int pos = a.token_pos[t];
   const int* table = a.block_tables + (size_t)a.token_seq[t] * a.max_blocks;
-  const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int reach = kv_reach(a, h0, nh);
+  const int lo =
+      max(0, pos - (a.window > 0 ? min(a.window, reach) : reach) + 1);
   const int nt = (pos - lo) / KV_TT + 1;
   const int hr = lane & 15, kq = lane >> 4;   // head row, key group
   const int head = h0 + min(hr, nh - 1);
@@ -408,9 +449,10 @@ __global__ __launch_bounds__(256, DK < 4 ? 4 : DK == 4 ? 3 : 1) void keyval_toke
   constexpr int NP = KV_TT * CPR / 64;      // per lane
   uint4 pre[NP];
   float fpre = 1.f;
-  // cache row of key (lane & 31) of a tile; rows past the last key repeat it
+  // tile n ends at position pos - 32 n; the last one may begin before lo, whose
+  // rows it repeats
   auto find = [&](int n) -> int {
-    const int j = min(lo + n * KV_TT + (lane & 31), pos);
+    const int j = max(pos - (n + 1) * KV_TT + 1 + (lane & 31), lo);
     return (table[j / a.BS] * a.G + g) * a.BS + (j % a.BS);
   };
   auto fetch = [&](int rowi) {
@@ -456,8 +498,8 @@ __global__ __launch_bounds__(256, DK < 4 ? 4 : DK == 4 ? 3 : 1) void keyval_toke
         st[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
             *(const kv_bf16x8*)(ka + 4 * x * PK + 32 * s), qr[s], st[x], 0, 0,
             0);
-    const int j0 = lo + n * KV_TT + 8 * kq;
-    const float base = sl2 * (float)(j0 - pos);
+    const int j0 = pos - (n + 1) * KV_TT + 1 + 8 * kq;
+    const float base = sl2 * (float)(j0 - pos) - (m == KV_LOW ? 0.f : m);
     float p[8], mx = -INFINITY;
 #pragma unroll
     for (int x = 0; x < 2; ++x) {
@@ -467,22 +509,15 @@ __global__ __launch_bounds__(256, DK < 4 ? 4 : DK == 4 ? 3 : 1) void keyval_toke
       for (int r = 0; r < 4; ++r) {
         const int i = 4 * x + r;
         p[i] = fmaf(st[x][r], f[r], fmaf(sl2, (float)i, base));
-        if (j0 + i > pos) p[i] = -INFINITY;
+        if (j0 + i < lo) p[i] = -INFINITY;
         mx = fmaxf(mx, p[i]);
       }
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float mnew = fmaxf(m, mx);
-    const float alpha = __builtin_amdgcn_exp2f(m - mnew);
-    l *= alpha;
-    m = mnew;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      p[i] = __builtin_amdgcn_exp2f(p[i] - mnew);
-      l += p[i];
-    }
-    if (__any(alpha != 1.f)) {
+    bool moved;
+    const float alpha = kv_softmax<8>(p, mx, &m, &l, &moved);
+    if (moved) {
 #pragma unroll
       for (int c = 0; c < NB; ++c)
 #pragma unroll
@@ -575,14 +610,15 @@ void mx_latent_combine(void* out, int ldout, const void* part, int T_, int H,
 
 // Returns 0 when launched, 1 when the shape is outside these kernels: rows of
 // whole 16-byte vectors, up to 256 entries. token: single tokens (every batch
-// row on its own), else prompt portions.
+// row on its own), else prompt portions. bound: of the scores' magnitude before
+// the distance penalty (0: unknown).
 int mx_keyval_attention(void* out, int ldout, const void* q, int ldq,
                         const void* rows, const void* kscale,
                         const void* block_tables, int max_blocks,
                         const void* token_seq, const void* token_pos, int T_,
                         int H, int G, int D, int BS, float scale, int window,
                         int sink, const void* sink_vals, const void* slopes,
-                        int token, int splits, void* scratch, void* stream) {
+                        float bound, int token, int splits, void* scratch, void* stream) {
   if (T_ <= 0) return 0;
   if (G < 1 || H < 1 || H % G || BS < 1 || D < 8 || D % 8 || D > 256 ||
       ldq % 8 || (((size_t)q | (size_t)rows) & 15))
@@ -593,7 +629,8 @@ int mx_keyval_attention(void* out, int ldout, const void* q, int ldq,
               (const float*)kscale, (const int*)block_tables, max_blocks,
               (const int*)token_seq, (const int*)token_pos, T_, H, G, D, BS,
               scale * KV_LOG2E, window, sink, (const float*)sink_vals,
-              (const float*)slopes, 1, nullptr, 0, 0};
+              (const float*)slopes, bound > 0.f ? bound * KV_LOG2E : -1.f, 1,
+              nullptr, 0, 0};
   if (!token) {
     a.hpb = rep < 128 ? rep : 128;
     a.hblocks = (rep + a.hpb - 1) / a.hpb;

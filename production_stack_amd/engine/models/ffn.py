@@ -239,11 +239,16 @@ class SparseMoE(nn.Module):
 
     def fused_in(self) -> torch.Tensor:
         """The shared expert's gate | up | scalar-gate rows as one weight;
-        the parts become views of it."""
+        the parts become views of it. Zero rows fill it up to a multiple of
+        64: the odd row count a scalar gate leaves behind would cost the
+        product its fast tiles and every reader its vector loads."""
         w = self._fused_in
         if w is None:
             parts = self.in_params()
-            w = torch.cat([p.data for p in parts], dim=0).contiguous()
+            pad = -sum(p.shape[0] for p in parts) % 64
+            w = torch.cat([p.data for p in parts]
+                          + [parts[0].data.new_zeros(pad, parts[0].shape[1])],
+                          dim=0).contiguous()
             off = 0
             for p in parts:
                 p.data = w[off:off + p.shape[0]]
@@ -325,6 +330,15 @@ class SparseMoE(nn.Module):
         act = self._act(gemm_policy.linear(xe, self.experts_gate_up[e]))
         return gemm_policy.linear(act, self.experts_down[e])
 
+    @staticmethod
+    def _gemm_rows(c: int) -> int:
+        """Rows of the product that runs an expert's c rows. The vendor
+        library looks for a kernel anew for every row count it has not met
+        (about 0.1 ms of host time, more than the product takes), so the
+        counts of large batches are rounded up to a few values."""
+        step = 128 if c <= 1024 else 256
+        return -(-c // step) * step
+
     @torch.no_grad()
     def _sorted_experts(self, x: torch.Tensor,
                         plan: ExpertPlan) -> torch.Tensor:
@@ -334,24 +348,33 @@ class SparseMoE(nn.Module):
         E = self.spec.experts
         counts = plan.host_counts()[:E]
         n = sum(counts)
-        xs = x.index_select(0, plan.rows[:n])
-        gu = torch.empty((n, self.experts_gate_up.shape[1]), dtype=x.dtype,
-                         device=x.device)
-        at = 0
-        for e, c in enumerate(counts):
-            if c:
-                torch.mm(xs[at:at + c], self.experts_gate_up[e].t(),
-                         out=gu[at:at + c])
-            at += c
+        # an expert's product may run past its rows into those of later
+        # experts (or the spare rows at the end), which come after it
+        spare = 256
+
+        def buf(cols: int) -> torch.Tensor:
+            return torch.empty((plan.rows.numel() + spare, cols),
+                               dtype=x.dtype, device=x.device)
+
+        def products(src, weight, dst) -> None:
+            at = 0
+            for e, c in enumerate(counts):
+                if c:
+                    m = self._gemm_rows(c) if x.is_cuda else c
+                    m = min(m, dst.shape[0] - at)
+                    torch.mm(src[at:at + m], weight[e].t(),
+                             out=dst[at:at + m])
+                at += c
+
+        xs = buf(x.shape[1])
+        torch.index_select(x, 0, plan.rows[:n], out=xs[:n])
+        gu = buf(self.experts_gate_up.shape[1])
+        products(xs, self.experts_gate_up, gu)
         act = self._act(gu)
-        ys = torch.empty((plan.rows.numel(), x.shape[1]), dtype=x.dtype,
-                         device=x.device)
-        at = 0
-        for e, c in enumerate(counts):
-            if c:
-                torch.mm(act[at:at + c], self.experts_down[e].t(),
-                         out=ys[at:at + c])
-            at += c
+        ys = buf(x.shape[1])
+        products(act, self.experts_down, ys)
+        # without the spare rows
+        ys = ys[:plan.rows.numel()]
         return ys
 
     def _grouped_fits(self, x: torch.Tensor) -> bool:
@@ -399,8 +422,8 @@ class SparseMoE(nn.Module):
                           plan: Optional[ExpertPlan] = None
                           ) -> torch.Tensor:
         """x: layer input [T, width]; proj: the shared expert's fused
-        projection [T, shared in-rows (+ 1 with a scalar gate)] (None
-        without a shared expert).
+        projection [T, shared in-rows (+ 1 with a scalar gate)], further
+        columns unused (None without a shared expert).
         dense=True insists on a path without a host read (what a captured
         decode step needs), None picks by batch size. plan: the step's
         routed rows, for table-routed layers. Returns fp32 [T, width]:
@@ -412,7 +435,7 @@ class SparseMoE(nn.Module):
             rows = self.shared.in_rows
             y = self.shared.forward_from_proj(proj[:, :rows])
             if self.shared_gate is not None:
-                gate = proj[:, rows:]
+                gate = proj[:, rows:rows + 1]
         if sp.score == "table":
             if plan is None:
                 raise ValueError("table-routed experts need the step's plan")

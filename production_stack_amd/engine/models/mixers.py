@@ -121,6 +121,9 @@ class TalkAttention(nn.Module):
             nn.Parameter(torch.empty((), dtype=torch.float32))
             if spec.v_mix else None)
         self._slopes = None
+        # unit-rms heads: |q . k| <= dim, with room for the queries' rounding
+        self.score_bound = (1.01 * abs(self.scale) * D if spec.unit_qk
+                            else 0.0)
 
     def in_params(self):
         return [self.qkv]
@@ -235,7 +238,8 @@ class TalkAttention(nn.Module):
                     talk=self.talk, out=out[a:b], variant=variant,
                     keep_first=sp.keep_first, softcap=sp.softcap,
                     sink_vals=self.sink_vals, pool=pool,
-                    key_scale=key_scale, slopes=self.slopes(proj.device))
+                    key_scale=key_scale, slopes=self.slopes(proj.device),
+                    score_bound=self.score_bound)
         if sp.out_gate:
             ops.gated_act(proj[:, self.qkv_rows:], out, "sigmoid", out=out)
         return out

@@ -624,7 +624,8 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
                    splits: int = 0, keep_first: int = 0,
                    softcap: float = 0.0, sink_vals: torch.Tensor = None,
                    vdim: int = 0, pool=None, key_scale: torch.Tensor = None,
-                   slopes: torch.Tensor = None) -> torch.Tensor:
+                   slopes: torch.Tensor = None,
+                   score_bound: float = 0.0) -> torch.Tensor:
     """Paged attention of a ragged batch. q [T, H*D] (row-strided view
     allowed); token_seq/token_pos int32 [T] give each token's block-table
     row and position; talk: optional fp32 [H, H] score mix; chunk/window:
@@ -640,6 +641,9 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
     BS]: the scores of a key are multiplied by its number; slopes fp32 [H]:
     slopes[h] * (query position - key position) is taken off the scaled
     scores (neither comes with a head mix, a cap or pooled blocks).
+    score_bound > 0: the caller knows that no scaled score exceeds it in
+    magnitude before the distance term; kernels may then pass over keys whose
+    weight is below 2^-40 of the largest one.
     variant 0 picks the kernel for prompt portions (tiled thread-per-
     (head, query) where the shape fits), 3 for single tokens (split-key),
     both falling back to the plain one-workgroup-per-token kernel; 1 / 2 /
@@ -745,7 +749,7 @@ def talk_attention(q: torch.Tensor, k_cache: torch.Tensor,
             _p(key_scale), _p(block_tables), block_tables.shape[1],
             _p(token_seq), _p(token_pos), T, H, G, D, BS, _f(scale),
             int(window), int(bool(sink)), _p(sink_vals), _p(slopes),
-            int(token), int(shares), _p(part), _stream())
+            _f(score_bound), int(token), int(shares), _p(part), _stream())
         if rc == 0:
             return out
     if variant in (8, 9):

@@ -75,8 +75,9 @@ def tune(weights, buckets, device) -> None:
 
 
 def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """F.linear with autotuned dispatch (no bias; Llama has none)."""
-    if x.is_cuda and _POLICY:
+    """F.linear with autotuned dispatch (no bias; Llama has none). The
+    in-house kernels are bfloat16 only; other types take the library."""
+    if x.is_cuda and _POLICY and x.dtype == torch.bfloat16:
         key = (x.shape[0], w.shape[0], w.shape[1])
         impl = _POLICY.get(key, 0)
         if impl:

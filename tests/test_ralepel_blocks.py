@@ -573,6 +573,50 @@ def test_keyval_prompt_kernel(shape):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("shape", [(2, 1, 8, 0), (8, 4, 128, 500),
+                                   (3, 3, 64, 0), (6, 2, 24, 40)])
+def test_known_score_bound_changes_nothing(shape):
+    """Unit queries and keys: with the bound given, keys beyond the reach of
+    every slope of a group are passed over; the result is the same, with and
+    without a window, at short and long distances."""
+    H, G, D, win = shape
+    lens, BS = [900, 1, 70, 333], 16
+    S = len(lens)
+    tables, rows, _ = page_setup(lens, G, D, BS, 7)
+    fac = 1.0 / rows.float().pow(2).mean(-1).sqrt()
+    slopes, sv = O.slopes(H).float(), rnd((H,), 3)
+    scale = D ** -0.5
+    for token in (True, False):
+        if token:
+            pos = torch.tensor([n - 1 for n in lens], dtype=torch.int32)
+            seq = torch.arange(S, dtype=torch.int32)
+        else:
+            pos = torch.cat([torch.arange(max(0, n - 150), n)
+                             for n in lens]).int()
+            seq = torch.cat([torch.full((min(n, 150),), i)
+                             for i, n in enumerate(lens)]).int()
+        T = len(pos)
+        q = rnd((T, H, D), 2)
+        q = (q / q.pow(2).mean(-1, keepdim=True).sqrt()).to(torch.bfloat16)
+        want = R.talk_attention(
+            q, rows, rows, tables, seq, pos, scale, 0, win, True, None, 0,
+            0.0, sv, D, None, fac, slopes).reshape(T, -1)
+        c = rows.cuda()
+        outs = [ops.talk_attention(
+            q.reshape(T, H * D).cuda(), c, c, tables.cuda(), seq.cuda(),
+            pos.cuda(), scale, H, window=win, sink=True, sink_vals=sv.cuda(),
+            vdim=D, variant=9 if token else 8, key_scale=fac.cuda(),
+            slopes=slopes.cuda(), score_bound=b)
+            for b in (0.0, 1.01 * scale * D)]
+        for o in outs:
+            err = (o.cpu().float() - want.float()).norm(dim=-1) / \
+                want.float().norm(dim=-1)
+            assert float(err.max()) < 1e-2, token
+        # the rounding of a result may fall either way, no more than that
+        assert relerr(*outs) < 1e-3
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("variant", [1, 2, 4])
 @pytest.mark.parametrize("shape", [(6, 2, 24, 20), (4, 1, 64, 0),
                                    (3, 3, 100, 33)])
