@@ -13,8 +13,10 @@
 //                   head: all its query heads of 128 / heads consecutive batch
 //                   rows, a wave 32 of them, so the heads of a group share
 //                   every staged tile. Queries stay in registers, 64 rows are
-//                   staged at a time, the next ones are on their way from
-//                   memory during the products. v_mfma_f32_32x32x16_bf16.
+//                   staged at a time in one of two LDS buffers, the next ones
+//                   are on their way from memory during the products and go
+//                   to the other buffer: one barrier per tile.
+//                   v_mfma_f32_32x32x16_bf16.
 //   token kernel    one (token, KV head, share of the rows) per workgroup,
 //                   and every wave on its own: 32 rows at a time into a
 //                   private piece of LDS, no workgroup barrier before the
@@ -39,6 +41,7 @@ typedef __attribute__((ext_vector_type(8))) __bf16 kv_bf16x8;
 typedef __attribute__((ext_vector_type(16))) float kv_f32x16;
 typedef __attribute__((ext_vector_type(4))) float kv_f32x4;
 typedef __attribute__((ext_vector_type(4))) short kv_s4;
+typedef __attribute__((ext_vector_type(4))) unsigned int kv_u4;
 typedef __attribute__((address_space(3))) kv_s4 kv_lds_s4;
 
 #define KV_LOG2E 1.44269504f
@@ -142,8 +145,8 @@ template <int DK, int OCC>
 __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
   constexpr int PK = DK * 16 + 8;
   constexpr int CB = DK / 2;        // 32-column blocks of the output
-  __shared__ __align__(16) unsigned short sR[KV_KT * PK];
-  __shared__ __align__(16) float s_f[KV_KT];
+  __shared__ __align__(16) unsigned short sR[2][KV_KT * PK];
+  __shared__ __align__(16) float s_f[2][KV_KT];
   __shared__ int s_row[2][KV_KT];
   __shared__ int s_seq[128], s_pos[128];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -202,14 +205,15 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
 
   constexpr int CPR = DK * 2;                  // 16-byte pieces per row
   constexpr int NP = KV_KT * CPR / 256;        // per thread
-  uint4 pre[NP];
+  kv_u4 pre[NP];
   float fpre = 0.f;
   // LDS row of this lane's key in a 32-key score tile
   const int krow = (row & 0x13) | ((row & 4) << 1) | ((row & 8) >> 1);
   const int i16 = lane & 15;
   // this lane's part of a transposed read
-  const unsigned short* va = sR + (8 * hi + (i16 >> 2)) * PK +
-                             16 * ((lane >> 4) & 1) + 4 * (i16 & 3);
+  const int vat = (8 * hi + (i16 >> 2)) * PK + 16 * ((lane >> 4) & 1) +
+                  4 * (i16 & 3);
+  const unsigned vis = a.window > 0 ? a.window : 0x7fffffff;
 
   int rs = 0;
   while (rs < ntok) {
@@ -225,7 +229,6 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
     const int nt = (kmax - kmin) / KV_KT + 1;
     // rows of other runs see nothing of this one
     const int pos = mine ? my_pos : -1;
-    const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
     // what the wave's rows of the run see: all of [w_full_lo, w_first], some
     // of [w_lo, w_last]
     const int ia = max(wave * 32 / HPB, rs);
@@ -235,42 +238,48 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
     const int w_lo = a.window > 0 ? max(0, w_first - a.window + 1) : 0;
     const int w_full_lo = a.window > 0 ? max(0, w_last - a.window + 1) : 0;
 
-    auto find = [&](int n, int buf) {
-      if (tid < KV_KT) {
-        // rows past the last key repeat it; they are masked
-        const int j = min(kmin + (nt - 1 - n) * KV_KT + tid, kmax);
-        s_row[buf][tid] = (table[j / a.BS] * a.G + g) * a.BS + (j % a.BS);
-      }
+    // page of row (tid & 63) of a tile; rows past the last key repeat it (they
+    // are masked). The page number is loaded well ahead of its use.
+    auto key_of = [&](int n) {
+      return min(kmin + (nt - 1 - n) * KV_KT + (tid & (KV_KT - 1)), kmax);
+    };
+    auto put_row = [&](int n, int page, int buf) {
+      if (tid < KV_KT)
+        s_row[buf][tid] = (page * a.G + g) * a.BS + key_of(n) % a.BS;
     };
     auto fetch = [&](int buf) {
+      int ri[NP];
+#pragma unroll
+      for (int u = 0; u < NP; ++u) ri[u] = s_row[buf][(u * 256 + tid) / CPR];
+      const int rf = s_row[buf][tid & (KV_KT - 1)];
 #pragma unroll
       for (int u = 0; u < NP; ++u) {
-        const int idx = u * 256 + tid;
-        const int r = idx / CPR, c = (idx - r * CPR) * 8;
-        pre[u] = c < D ? *(const uint4*)(a.rows +
-                                         (int64_t)s_row[buf][r] * D + c)
-                       : make_uint4(0, 0, 0, 0);
+        // columns past the row's end repeat its last piece: finite numbers
+        // that meet zero query entries or land in columns never stored
+        const int c = min((u * 256 + tid) % CPR * 8, D - 8);
+        pre[u] = *(const kv_u4*)(a.rows + (int64_t)ri[u] * D + c);
       }
-      if (tid < KV_KT)
-        fpre = a.kscale != nullptr ? a.kscale[s_row[buf][tid]] : 1.f;
+      fpre = a.kscale != nullptr ? a.kscale[rf] : 1.f;
     };
-    find(0, 0);
-    if (nt > 1) find(1, 1);
-    __syncthreads();
-    fetch(0);
+    put_row(0, table[key_of(0) / a.BS], 1);
+    __syncthreads();  // also: the previous run's tiles are fully read
+    fetch(1);
+    int page = table[key_of(min(1, nt - 1)) / a.BS];
     for (int n = 0; n < nt; ++n) {
-      __syncthreads();  // the previous tile is fully read
+      // tile n from registers to its buffer, which tile n - 2 has left; what
+      // lies past the last tile repeats it
 #pragma unroll
       for (int u = 0; u < NP; ++u) {
         const int idx = u * 256 + tid;
-        const int r = idx / CPR, c = (idx - r * CPR) * 8;
-        *(uint4*)(sR + r * PK + c) = pre[u];
+        *(kv_u4*)(&sR[n & 1][idx / CPR * PK + idx % CPR * 8]) = pre[u];
       }
-      if (tid < KV_KT) s_f[tid] = fpre * a.scale2;
-      // buffer n & 1 held this tile's rows, which are all fetched
-      if (n + 2 < nt) find(n + 2, n & 1);
+      if (tid < KV_KT) s_f[n & 1][tid] = fpre * a.scale2;
+      put_row(min(n + 1, nt - 1), page, n & 1);
       __syncthreads();
-      if (n + 1 < nt) fetch((n + 1) & 1);
+      fetch(n & 1);
+      page = table[key_of(min(n + 2, nt - 1)) / a.BS];
+      const unsigned short* sr = sR[n & 1];
+      const float* sf = s_f[n & 1];
       const int j0 = kmin + (nt - 1 - n) * KV_KT;
       if (!live || j0 > w_last || j0 + KV_KT - 1 < w_lo) continue;
 
@@ -279,7 +288,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
       for (int r = 0; r < 16; ++r) st[0][r] = st[1][r] = 0.f;
 #pragma unroll
       for (int s = 0; s < DK; ++s) {
-        const unsigned short* ka = sR + krow * PK + 16 * s + 8 * hi;
+        const unsigned short* ka = sr + krow * PK + 16 * s + 8 * hi;
         const kv_bf16x8 a0 = *(const kv_bf16x8*)ka;
         const kv_bf16x8 a1 = *(const kv_bf16x8*)(ka + 32 * PK);
         st[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a0, qr[s], st[0], 0,
@@ -295,9 +304,9 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
       for (int h = 0; h < 2; ++h)
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-          const float4 f0 = *(const float4*)(s_f + 32 * h + 16 * s + 8 * hi);
+          const float4 f0 = *(const float4*)(sf + 32 * h + 16 * s + 8 * hi);
           const float4 f1 =
-              *(const float4*)(s_f + 32 * h + 16 * s + 8 * hi + 4);
+              *(const float4*)(sf + 32 * h + 16 * s + 8 * hi + 4);
           const float f[8] = {f0.x, f0.y, f0.z, f0.w, f1.x, f1.y, f1.z, f1.w};
 #pragma unroll
           for (int i = 0; i < 8; ++i)
@@ -305,13 +314,15 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
                 fmaf(st[h][8 * s + i], f[i],
                      fmaf(sl2, (float)(32 * h + 16 * s + i), base));
         }
+      const int dist = pos - j0 - 8 * hi;  // of this lane's first key
       if (!all_mine || j0 < w_full_lo || j0 + KV_KT - 1 > w_first) {
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
-            const int j = j0 + 32 * h + 16 * (r >> 3) + 8 * hi + (r & 7);
-            if (j > pos || j < lo) w[16 * h + r] = -INFINITY;
+            // a distance below zero (a later key) is a huge unsigned number
+            const int d = dist - (32 * h + 16 * (r >> 3) + (r & 7));
+            if ((unsigned)d >= vis) w[16 * h + r] = -INFINITY;
           }
       }
       float mx = w[0];
@@ -339,7 +350,7 @@ __global__ __launch_bounds__(256, OCC) void keyval_prompt_kernel(KvArgs a) {
 #pragma unroll
           for (int h = 0; h < 2; ++h)
             v.h[h] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                (kv_lds_s4*)(va + (16 * s + 4 * h) * PK + 32 * c));
+                (kv_lds_s4*)(sr + vat + (16 * s + 4 * h) * PK + 32 * c));
           acc[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v.v, b0.v, acc[c],
                                                            0, 0, 0);
           acc[c] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v.v, b1.v, acc[c],
